@@ -9,8 +9,9 @@ table [max_rows, table_width] that all slots of a group share.
 Beyond the reference: cache slots are collected into *groups* by what they need
 (all keys, or a window of them; a page shape); each group has its own allocator,
 table and pools. Pages are taken when a step needs them, not reserved at
-admission, and given back when a row closes or, in a windowed group, when every
-position of a page lies behind the window of every token still to come. Mixers
+admission, and given back when a row closes or, in a group with a window or with
+chunks, when every position of a page lies behind the window (or in a chunk before
+that) of every token still to come. Mixers
 with a state of fixed size get a float32 tensor [max_rows, *shape] per slot,
 cleared when a row opens. Fixed-size per-request scalars (length, sampling
 parameters, counters) live in ``RowScalars``.
@@ -86,9 +87,10 @@ class PagedGroup:
     # -- pages a row needs / can drop ---------------------------------------------------------
     def droppable(self, row: int, next_start: int) -> int:
         """Logical blocks of ``row`` that no token at position >= next_start can see."""
-        if self.need.window is None or self.means:
+        chunk = getattr(self.need, "chunk", None)
+        if (self.need.window is None and chunk is None) or self.means:
             return self.first_live[row]
-        first_visible = max(0, next_start - self.need.window + 1)
+        first_visible = next_start // chunk * chunk if chunk is not None else max(0, next_start - self.need.window + 1)
         pool = getattr(self.need, "pool", 0)
         if pool:
             # the block that holds next_start is not complete: its tokens stay until its mean is taken
@@ -220,6 +222,9 @@ class CacheManager:
             pool = getattr(need, "pool", 0)
             if pool < 0 or (pool and (need.window is None or need.keep_first)):
                 raise ValueError("pooled blocks need a window, and no kept first positions")
+            chunk = getattr(need, "chunk", None)
+            if chunk is not None and (chunk < 1 or need.window is not None or getattr(need, "keep_first", 0)):
+                raise ValueError("chunks hold at least one position and take the place of a window")
             group = self._group(need, need, self._num_blocks)
             serial = len(group.pools)
             group.add_slot(serial)

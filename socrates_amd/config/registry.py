@@ -13,6 +13,7 @@ from pathlib import Path
 
 from .berelorn import BerelornConfig
 from .mitisun import MitisunConfig
+from .nebutar import NebutarConfig
 from .pozalorn import PozalornConfig
 from .qwen3 import ConfigError, Qwen3Config
 from .sovezen import SovezenConfig
@@ -106,3 +107,4 @@ register_architecture("Tedulorn", TedulornConfig)
 register_architecture("Pozalorn", PozalornConfig)
 register_architecture("Berelorn", BerelornConfig)
 register_architecture("Sovezen", SovezenConfig)
+register_architecture("Nebutar", NebutarConfig)

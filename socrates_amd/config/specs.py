@@ -23,6 +23,14 @@ class RMSNormSpec:
 
 
 @dataclass(frozen=True)
+class LayerNormSpec:
+    """y = (x - mean) / sqrt(variance + eps) * w + b over the last ``dim`` elements, the variance being the mean of
+    the squared deviations. w carries the norm's own name on disk, b that name with ``.b`` behind it."""
+    dim: int
+    eps: float
+
+
+@dataclass(frozen=True)
 class RopeSpec:
     """Rotate-half rotary encoding over the first ``rotary_dim`` of each head.
 
@@ -379,7 +387,10 @@ class RoutedExpertsSpec:
     (``router.b``) is added to the logits ahead of everything. ``group_top`` = n: a group's score is the
     sum of its n largest choice scores (1: its largest). ``scale``: the weights are multiplied by it. ``expert`` and
     ``shared`` may also be a ``SwiGLUSpec`` (a plain silu gate, no clamp), ``expert`` also a ``ReluSquaredSpec``. ``shared_gate``: the shared expert's
-    result is multiplied by sigmoid(w_sg . x), one number per token (stored as ``shared.sg`` [1, hidden])."""
+    result is multiplied by sigmoid(w_sg . x), one number per token (stored as ``shared.sg`` [1, hidden]).
+
+    ``renorm`` False (softmax or sigmoid scores): the weights are the chosen experts' s as they are. ``n_identity``: the
+    last that many of the ``n_experts`` outputs of the router are experts without tensors, whose result is the input."""
     hidden: int
     n_experts: int
     top: int
@@ -394,8 +405,14 @@ class RoutedExpertsSpec:
     scale: float = 1.0
     shared_gate: bool = False
     logit_bias: bool = False
+    renorm: bool = True
+    n_identity: int = 0
 
     def __post_init__(self):
+        if not 0 <= self.n_identity < self.n_experts:
+            raise ValueError(f"{self.n_identity} of {self.n_experts} experts are identity experts")
+        if self.scoring == "chosen" and not self.renorm:
+            raise ValueError("a softmax over the chosen logits has its own sum")
         if self.scoring not in ("softmax", "sigmoid", "chosen"):
             raise ValueError(f"scoring {self.scoring!r}: softmax, sigmoid or chosen")
         if self.scoring == "chosen" and self.renorm_eps != 0.0:
@@ -444,7 +461,8 @@ class WindowAttentionSpec:
     ``tied_values``: there is no value projection; a token's values are its keys as projected, before norm and
     rotation (v_dim equals head_dim). ``softcap`` = c: a scaled score s becomes c tanh(s / c). ``head_gate``: head
     h's result is multiplied by sigmoid(W_g x)_h (stored as ``g`` [heads, hidden]) before the output projection.
-    ``keep_first``: with a window, the keys at positions below it stay visible to every later token."""
+    ``keep_first``: with a window, the keys at positions below it stay visible to every later token. ``chunk`` = c
+    (in place of a window): a query at position i sees key j <= i only if floor(i / c) = floor(j / c)."""
     hidden: int
     n_heads: int
     n_kv_heads: int
@@ -464,12 +482,15 @@ class WindowAttentionSpec:
     softcap: Optional[float] = None
     head_gate: bool = False
     keep_first: int = 0
+    chunk: Optional[int] = None
 
     def __post_init__(self):
         if self.n_heads < 1 or self.n_kv_heads < 1 or self.n_heads % self.n_kv_heads:
             raise ValueError(f"n_heads {self.n_heads} is not a multiple of n_kv_heads {self.n_kv_heads}")
         if not 1 <= self.head_dim <= 256 or not 1 <= self.v_dim <= 256:
             raise ValueError(f"head sizes {self.head_dim} and {self.v_dim}: the attention kernels take up to 256")
+        if self.chunk is not None and (self.chunk < 1 or self.window is not None or self.keep_first):
+            raise ValueError("chunks hold at least one position and take the place of a window and its kept first keys")
         if self.qk_norm not in (None, "head", "whole", "turned"):
             raise ValueError(f"qk_norm {self.qk_norm!r}: head, whole, turned or None")
         if self.window is not None and self.window < 1:
@@ -622,6 +643,37 @@ class LightningAttentionSpec:
 
 
 @dataclass(frozen=True)
+class GatedDeltaSpec:
+    """Gated delta rule: a matrix state per head that forgets by a scalar and corrects what it holds for a key. q, k
+    [``n_kv_heads`` x ``head_dim``] and v [``n_heads`` x ``v_dim``] each pass a causal convolution of ``conv_taps`` taps per
+    channel and silu; q and k become unit vectors per head, x / sqrt(sum(x^2) + ``unit_eps``), q also times
+    head_dim^-1/2; head h uses q / k head floor(h / (n_heads / n_kv_heads)). beta = sigmoid(W_b h),
+    g = exp(-exp(A_log) softplus(W_a h + dt_bias)), one each per head. S <- g S; u = beta (v - S^T k);
+    S <- S + k u^T; o = S^T q. Each head's o over its root mean square (eps), times one gain of v_dim for all heads,
+    times silu(W_g h), then the output projection. The state is float32 and starts at zero."""
+    hidden: int
+    n_heads: int
+    n_kv_heads: int
+    head_dim: int
+    v_dim: int
+    conv_taps: int
+    eps: float
+    unit_eps: float = 1e-6
+
+    def __post_init__(self):
+        if self.n_heads < 1 or self.n_kv_heads < 1 or self.n_heads % self.n_kv_heads:
+            raise ValueError(f"n_heads {self.n_heads} is not a multiple of n_kv_heads {self.n_kv_heads}")
+        if not 1 <= self.head_dim <= 256 or self.v_dim < 1:
+            raise ValueError(f"gated delta rule: heads of {self.head_dim} (1 to 256) and {self.v_dim}")
+        if not 1 <= self.conv_taps <= 33:
+            raise ValueError(f"gated delta rule: a convolution of {self.conv_taps} taps (1 to 33)")
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.n_kv_heads * self.head_dim + self.n_heads * self.v_dim
+
+
+@dataclass(frozen=True)
 class ParallelMixerSpec:
     """Two mixers side by side on the same input: ``left_scale`` * left(h) + ``right_scale`` * right(h);
     their tensors lie under ``left.`` and ``right.``, and each keeps its own cache or state."""
@@ -653,6 +705,20 @@ class DepthAverageSpec:
     ``n_layers``: how many layers the model has (a step keeps that many results and one)."""
     index: int
     n_layers: int
+
+
+@dataclass(frozen=True)
+class StreamsSpec:
+    """How a branch reads and writes ``n`` copies x_1 .. x_n of the residual stream: it reads u = sum_s in[s] x_s, and
+    with y its result x_t <- sum_s mix[s, t] x_s + out[t] y, all t at once (stored: ``in`` [n], ``mix`` [n, n],
+    ``out`` [n])."""
+    n: int
+
+    MAX_STREAMS = 16
+
+    def __post_init__(self):
+        if not 1 <= self.n <= self.MAX_STREAMS:
+            raise ValueError(f"{self.n} copies of the stream (1 to {self.MAX_STREAMS})")
 
 
 @dataclass(frozen=True)
@@ -693,8 +759,14 @@ class BlockSpec:
     # by one).
     scale1: object = None
     scale2: object = None
+    # For the arrangement "streams": the residual is several copies of the stream (``ModelPlan.streams``); the mixer
+    # reads and writes them through ``streams1``, the feed-forward through ``streams2`` (a ``StreamsSpec`` each): u from
+    # the copies, y = branch(norm(u)), then the copies from the old copies and y. (``ffn`` None: no norm2, no streams2.)
+    streams1: object = None
+    streams2: object = None
 
-    ROLES = ("norm1", "mixer", "norm2", "ffn", "post_norm1", "post_norm2", "gate1", "gate2", "side", "depth", "scale1", "scale2")
+    ROLES = ("norm1", "mixer", "norm2", "ffn", "post_norm1", "post_norm2", "gate1", "gate2", "side", "depth", "scale1", "scale2",
+             "streams1", "streams2")
 
     def name_of(self, role: str) -> str:
         return self.prefix + dict(self.names)[role]
@@ -736,10 +808,22 @@ class ModelPlan:
     embedding_scale: float = 1.0
     logit_scale: float = 1.0
     logit_softcap: Optional[float] = None
+    # learned positions: the name of a table [max_positions, hidden] whose row p is added to the (scaled) embedding of
+    # the token at position p; no sequence is longer than the table
+    positions_name: Optional[str] = None
+    max_positions: Optional[int] = None
+    # copies of the residual stream (None: one stream, [tokens, hidden]); with n of them the stream is [tokens, n,
+    # hidden], every copy starts as the embedding's output, and their sum goes to the final norm
+    streams: Optional[int] = None
 
     def __post_init__(self):
         if self.logit_softcap is not None and not self.logit_softcap > 0:
             raise ValueError("logit_softcap must be positive")
+        if (self.positions_name is None) != (self.max_positions is None):
+            raise ValueError("a table of positions comes with its length")
+        for block in self.layers:
+            if (block.arrangement == "streams") != (self.streams is not None):
+                raise ValueError("blocks of the arrangement 'streams' and a plan with copies of the stream come together")
         written = set()
         for step in self.order:
             if not 0 <= step.layer < len(self.layers):

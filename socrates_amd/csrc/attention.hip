@@ -80,6 +80,14 @@ struct ScoreTerms {
     int pool;
 };
 
+// The first key that a token at position p sees: 0 without a window (window == 0), p - window + 1 behind a sliding
+// window, and with window < 0 the first position of the token's chunk: chunks of -window positions, counted from
+// position 0 of the sequence.
+__device__ __forceinline__ int first_seen(int p, int window) {
+    if (window > 0) return max(0, p - window + 1);
+    return window < 0 ? p - p % -window : 0;
+}
+
 // How many entries a token at position p walks before its window (which starts at lo): kept first keys, or the
 // means of the blocks that end before the window begins.
 __device__ __forceinline__ int walk_prefix(const ScoreTerms& st, int p, int window, int lo) {
@@ -100,7 +108,7 @@ paged_attn_token_kernel(const T* __restrict__ q, const T* __restrict__ k_pool,
     const int kvh = blockIdx.x / chunks, g0 = (blockIdx.x % chunks) * GC;
     const int n = blockIdx.y, split = blockIdx.z;
     const int p = positions[n];
-    const int lo = window > 0 ? max(0, p - window + 1) : 0;
+    const int lo = first_seen(p, window);
     const int kf = walk_prefix(st, p, window, lo);     // kept first keys (or means of blocks) that lie before the window
     // the token's keys in the order they are walked: the kept first ones, then lo .. p
     const int start = split * split_len;
@@ -235,7 +243,7 @@ __global__ void paged_attn_reduce_kernel(const float* __restrict__ part_o,
                                          int Hq, int window, int split_len, int n_splits, ScoreTerms st) {
     const int h = blockIdx.x, n = blockIdx.y;
     const int p = positions[n];
-    const int lo = window > 0 ? max(0, p - window + 1) : 0;
+    const int lo = first_seen(p, window);
     const int np = min(n_splits, (walk_prefix(st, p, window, lo) + p + 1 - lo + split_len - 1) / split_len);
     const size_t base = ((size_t)n * Hq + h) * n_splits;
     float M = st.sinks ? st.sinks[h] : -INFINITY;
@@ -283,7 +291,7 @@ static int dispatch_token(int G, const void* q, const void* k_pool, const void* 
 #undef SOC_ARGS
 }
 
-// q [N, Hq, D]; pools [pages, Hkv, BS, D]; out [N, Hq, D]. window <= 0: no window.
+// q [N, Hq, D]; pools [pages, Hkv, BS, D]; out [N, Hq, D]. window 0: no window; < 0: chunks of -window positions.
 // n_splits > 1 needs part_o [N, Hq, n_splits, D] and part_ml [N, Hq, n_splits, 2] (float32);
 // split s covers the keys s * split_len .. of each token's walk (the kept first keys, then its window).
 // softcap (0: none), sinks and slopes ([Hq] float32 each, or null) and keep_first (0: none): see
@@ -455,7 +463,7 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_po
     // for: no wave of a short row walks far, none of a long row is idle
     int split_len = split_len_arg, first_key = 0;
     if (split_len_arg <= 0) {
-        first_key = window > 0 ? max(0, pos0 - window + 1) & ~15 : 0;
+        first_key = first_seen(pos0, window) & ~15;
         split_len = max(16, ((pos0 + ntok - first_key + n_splits - 1) / n_splits + 15) & ~15);
     }
     const int split_lo = first_key + split * split_len;     // the split's first key
@@ -464,14 +472,14 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_po
     const bool own_key = FUSED && fz.write_kv;
     const bool covers = pos0 >= klo && pos0 < klo + split_len;      // this wave's split holds the token's position
     int khi = min(klo + split_len, own_key ? pos0 : pos0 + ntok);
-    if (window > 0) klo = max(klo, pos0 - window + 1);
+    klo = max(klo, first_seen(pos0, window));
     const int kmin = klo;                                // first key any row of the block can see
     klo = klo & ~15;                                     // tiles are aligned to 16 keys
     const int li = lane % 16, kb = lane / 16;
     uint16_t* vl = v_lds[wave];
 
     // rows of this lane's column, per row tile
-    int row_pos[RT];                                     // position of the row's token, -1: no row
+    int row_pos[RT], row_first[RT];                      // position of the row's token (-1: no row), the first key it sees
     size_t row_q[RT];                                    // offset of the row's query / output
     uint4 qf[RT][QK_STEPS];
 #pragma unroll
@@ -480,6 +488,7 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_po
         const int tt = rho >> group_pad_log2, g = chunk * 16 + (rho & (Gp - 1));
         const bool ok = tt < ntok && g < G;
         row_pos[rt] = ok ? pos0 + tt : -1;
+        row_first[rt] = first_seen(ok ? pos0 + tt : pos0, window);
         row_q[rt] = ((size_t)(tok0 + (ok ? tt : 0)) * Hq + (size_t)kvh * G + (ok ? g : 0)) * D;
         if constexpr (!FUSED) {
 #pragma unroll
@@ -705,7 +714,7 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_po
                 if constexpr (MASKED) {
                     const int key = key0 + 4 * kb + r;
                     bool seen = key <= row_pos[rt] && key < hi && key >= lo_seen;
-                    if (window > 0) seen = seen && key > row_pos[rt] - window;
+                    if (window != 0) seen = seen && key >= row_first[rt];
                     sv[r] = seen ? sv[r] : -INFINITY;
                 }
                 mx = fmaxf(mx, sv[r]);
@@ -749,10 +758,10 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_po
     };
     // whole: every key of the tile lies in the split, at or before the block's first position
     // and inside the window of its last one, so no score needs a mask
-    const int last_pos = pos0 + ntok - 1;
+    const int last_first = first_seen(pos0 + ntok - 1, window);
     auto tile = [&](int key0, const KFrag& kf, const uint4 (&vr)[V_PER_LANE]) {
         const bool whole = key0 >= split_lo && key0 + 15 < khi && key0 + 15 <= pos0 &&
-                           (window <= 0 || key0 > last_pos - window);
+                           key0 >= last_first;
         s16x4_t pf[RT];
         float alpha[RT];
         bool any_rescale;
@@ -1172,7 +1181,7 @@ paged_attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k
     const int tokens_per_wave = ((M32 ? 32 : 16 * RT)) >> group_pad_log2;
 
     const int khi = pos0 + ntok;                                    // keys any row of the block sees
-    int kmin = window > 0 ? max(0, pos0 - window + 1) : 0;
+    int kmin = first_seen(pos0, window);
     // With a window, the keys below keep_first stay visible. Those of them that lie before the window of the
     // block's first row (kept of them) are walked first, in tiles of their own that stand in front of the
     // window's tiles (n_pre of them, the walk then starts at the virtual key klo - n_pre * PF_KEYS); where
@@ -1206,12 +1215,13 @@ paged_attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k
     const int wave_lo_pos = pos0 + wtok0;                           // its first and last positions
     const int wave_hi_pos = min(khi, wave_lo_pos + tokens_per_wave) - 1;
     const bool wave_has_rows = wtok0 < ntok;
+    const int wave_first = first_seen(wave_hi_pos, window);         // the first key that all of the wave's rows see
     const float c2 = scale * 1.44269504088896340736f;               // to base 2
     const SoftCap capped(scale, softcap);
     const int means_lo = pool > 0 ? blocks_before(wave_lo_pos) : 0; // entries that all / any of the wave's rows see
     const int means_hi = pool > 0 ? blocks_before(wave_hi_pos) : 0;
 
-    int row_pos[RT], mean_end[RT];                                  // (mean_end: the first entry of means a row does not see)
+    int row_pos[RT], row_first[RT], mean_end[RT];                   // (mean_end: the first entry of means a row does not see)
     float sink_l2[RT];                                              // a learned sink (sink == 2), to base 2
     size_t row_q[RT];
     uint4 qf[RT][QK_STEPS];
@@ -1221,6 +1231,7 @@ paged_attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k
         const int tt = wtok0 + (rho >> group_pad_log2), g = chunk * 16 + (rho & (Gp - 1));
         const bool ok = tt < ntok && g < G;
         row_pos[rt] = ok ? pos0 + tt : -1;
+        row_first[rt] = first_seen(ok ? pos0 + tt : pos0, window);
         row_q[rt] = ((size_t)(tok0 + (ok ? tt : 0)) * Hq + (size_t)kvh * G + (ok ? g : 0)) * D;
         mean_end[rt] = PF_MEAN + (pool > 0 && ok ? blocks_before(pos0 + tt) : 0);
         sink_l2[rt] = sink == 2 && ok ? sinks[kvh * G + g] * 1.44269504088896340736f : 0.f;
@@ -1239,7 +1250,7 @@ paged_attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k
     // 32-row products: the lane's row is lane % 32, its half of every 16-wide k step lane / 32
     constexpr int DQ32 = D / 16, DB32 = D / 32;
     const int c32 = lane % 32, g32 = lane / 32;
-    int row_pos32 = -1, mean_end32 = PF_MEAN;
+    int row_pos32 = -1, row_first32 = 0, mean_end32 = PF_MEAN;
     float sink32_l2 = 0.f;
     size_t row_q32 = 0;
     uint4 qf32[M32 ? DQ32 : 1];                           // the lane's slices of its query row
@@ -1249,6 +1260,7 @@ paged_attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k
         const int tt = wtok0 + (c32 >> group_pad_log2), gh = chunk * 16 + (c32 & (Gp - 1));
         const bool ok = tt < ntok && gh < G;
         row_pos32 = ok ? pos0 + tt : -1;
+        row_first32 = first_seen(ok ? pos0 + tt : pos0, window);
         row_q32 = ((size_t)(tok0 + (ok ? tt : 0)) * Hq + (size_t)kvh * G + (ok ? gh : 0)) * D;
         if (pool > 0 && ok) mean_end32 = PF_MEAN + blocks_before(pos0 + tt);
         if (sink == 2 && ok) sink32_l2 = sinks[kvh * G + gh] * 1.44269504088896340736f;
@@ -1377,7 +1389,7 @@ paged_attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k
                 if constexpr (MASKED) {
                     const int key = key0 + 8 * kb + r;
                     bool seen = key <= row_pos[rt];
-                    if (window > 0) seen = seen && (key > row_pos[rt] - window || key < keep_first);
+                    if (window != 0) seen = seen && (key >= row_first[rt] || key < keep_first);
                     if (key0 < 0) seen = key < mean_end[rt];          // (uniform: a tile of means)
                     t[r] = seen ? t[r] : -INFINITY;
                 }
@@ -1448,7 +1460,7 @@ paged_attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k
             if constexpr (MASKED) {
                 const int key = key0 + 16 * (i / 8) + 8 * g32 + i % 8;
                 bool seen = key <= row_pos32;
-                if (window > 0) seen = seen && (key > row_pos32 - window || key < keep_first);
+                if (window != 0) seen = seen && (key >= row_first32 || key < keep_first);
                 if (key0 < 0) seen = key < mean_end32;               // (uniform: a tile of means)
                 sc[i] = seen ? sc[i] : -INFINITY;
             }
@@ -1519,7 +1531,7 @@ paged_attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k
             // whole: every key of the tile is at or before the wave's first position and inside
             // the window of its last one (of means: all its entries are seen by the wave's first row)
             const bool whole = of_means ? key0 - PF_MEAN + PF_KEYS <= means_lo
-                                        : key0 + PF_KEYS - 1 <= wave_lo_pos && (window <= 0 || key0 > wave_hi_pos - window);
+                                        : key0 + PF_KEYS - 1 <= wave_lo_pos && key0 >= wave_first;
             if constexpr (M32) {
                 uint4 pf[2];
                 float alpha;

@@ -350,7 +350,7 @@ SOC_EXPORT int soc_relu_squared(const void* x, void* out, long long total, int d
 // keep_groups best groups can be chosen (n_groups <= 1: all). The top experts by c (the lower index among
 // equals) are chosen; their weights are their s over the sum of the chosen s (+ renorm_eps). bias (if given) is added
 // to z first. scoring 0: softmax, 1: sigmoid, 2: c = z itself (+ correction), s = exp(z - the largest z), so that the
-// weights are the softmax over the chosen logits.
+// weights are the softmax over the chosen logits. renorm 0: the weights are the chosen experts' s as they are.
 __device__ __forceinline__ void wave_argmax(float& v, int& i) {
 #pragma unroll
     for (int m = 32; m >= 1; m >>= 1) {
@@ -362,8 +362,8 @@ __device__ __forceinline__ void wave_argmax(float& v, int& i) {
 
 __global__ void __launch_bounds__(256)
 moe_route_kernel(const float* __restrict__ z, int ldz, const float* __restrict__ bias, const float* __restrict__ correction, int N, int E,
-                 int top, int n_groups, int keep_groups, float renorm_eps, int scoring, int group_top, float scale, int* __restrict__ idx,
-                 float* __restrict__ weight) {
+                 int top, int n_groups, int keep_groups, float renorm_eps, int scoring, int group_top, float scale, int renorm,
+                 int* __restrict__ idx, float* __restrict__ weight) {
     __shared__ float sc[4][256];
     __shared__ float ss[4][256];
     const int wave = threadIdx.x / SOC_WAVE, lane = threadIdx.x % SOC_WAVE;
@@ -472,18 +472,18 @@ moe_route_kernel(const float* __restrict__ z, int ldz, const float* __restrict__
         if (lane == 0) { idx[(size_t)n * top + r] = bi; sc[wave][r] = ss[wave][bi]; }     // (sc is free: cv holds it)
     }
     if (lane == 0)
-        for (int r = 0; r < top; ++r) weight[(size_t)n * top + r] = sc[wave][r] / (total + renorm_eps) * scale;
+        for (int r = 0; r < top; ++r) weight[(size_t)n * top + r] = (renorm ? sc[wave][r] / (total + renorm_eps) : sc[wave][r]) * scale;
 }
 
 SOC_EXPORT int soc_moe_route(const float* z, int ldz, const float* bias, const float* correction, int N, int E, int top, int n_groups,
-                             int keep_groups, float renorm_eps, int scoring, int group_top, float scale, int* idx, float* weight,
-                             hipStream_t stream) {
+                             int keep_groups, float renorm_eps, int scoring, int group_top, float scale, int renorm, int* idx,
+                             float* weight, hipStream_t stream) {
     if (N <= 0) return 0;
     if (E < 1 || E > 256 || ldz < E || scoring < 0 || scoring > 2 || group_top < 1 || top < 1 || top > E || n_groups < 1 || E % n_groups || keep_groups < 1 || keep_groups > n_groups ||
         (long long)keep_groups * (E / n_groups) < top)
         return (int)hipErrorInvalidValue;
     hipLaunchKernelGGL(moe_route_kernel, dim3((N + 3) / 4), dim3(256), 0, stream, z, ldz, bias, correction, N, E, top, n_groups,
-                       keep_groups, renorm_eps, scoring, group_top, scale, idx, weight);
+                       keep_groups, renorm_eps, scoring, group_top, scale, renorm, idx, weight);
     return soc_last_error();
 }
 
@@ -491,7 +491,8 @@ SOC_EXPORT int soc_moe_route(const float* z, int ldz, const float* bias, const f
 // idx [M] (M = tokens x top): the expert of each (token, choice) pair. One workgroup counts the pairs of each
 // expert, lays the experts' runs one after the other (offsets [E + 1]), gives each pair its place (place [M]) and
 // each place its pair (pair_at [M]), and lists the tiles of TM places that the products walk: tiles [max_tiles, 2]
-// = (expert, first place), expert -1 behind the last tile. max_tiles >= M / TM + E.
+// = (expert, first place), expert -1 behind the last tile. max_tiles >= M / TM + E. A pair whose expert is E or more (an
+// identity expert: nothing to compute) gets no place: -1.
 __global__ void __launch_bounds__(1024)
 moe_sort_kernel(const int* __restrict__ idx, int M, int E, int TM, int max_tiles, int* __restrict__ offsets,
                 int* __restrict__ place, int* __restrict__ pair_at, int* __restrict__ tiles) {
@@ -499,7 +500,8 @@ moe_sort_kernel(const int* __restrict__ idx, int M, int E, int TM, int max_tiles
     const int tid = threadIdx.x;
     for (int e = tid; e < E; e += 1024) count[e] = 0;
     __syncthreads();
-    for (int i = tid; i < M; i += 1024) atomicAdd(&count[idx[i]], 1);
+    for (int i = tid; i < M; i += 1024)
+        if (idx[i] < E) atomicAdd(&count[idx[i]], 1);
     __syncthreads();
     if (tid == 0) {
         int at = 0, t = 0;
@@ -515,6 +517,7 @@ moe_sort_kernel(const int* __restrict__ idx, int M, int E, int TM, int max_tiles
     for (int e = tid; e < E; e += 1024) cursor[e] = start[e];
     __syncthreads();
     for (int i = tid; i < M; i += 1024) {
+        if (idx[i] >= E) { place[i] = -1; continue; }
         const int at = atomicAdd(&cursor[idx[i]], 1);
         place[i] = at;
         pair_at[at] = i;
@@ -789,30 +792,32 @@ SOC_EXPORT int soc_grouped_linear(const void* x, int ldx, const int* pair_at, in
 
 // ---- the weighted sum of a token's experts ---------------------------------------------------------------------------
 // out[n, c] = sum_r weight[n, r] y[place[n top + r], c] (+ extra[n, c], times sigmoid(gate[n ldg]) if gate is given), float32;
-// y float32 [M, d] by place.
+// y float32 [M, d] by place; a place below 0 stands for row n of through (compute dtype, [N, d]).
 template <typename T>
 __global__ void moe_combine_kernel(const float* __restrict__ y, const int* __restrict__ place, const float* __restrict__ weight,
-                                   const T* __restrict__ extra, const float* __restrict__ gate, int ldg, float* __restrict__ out,
-                                   int N, int d, int top) {
+                                   const T* __restrict__ extra, const float* __restrict__ gate, int ldg, const T* __restrict__ through,
+                                   float* __restrict__ out, int N, int d, int top) {
     const int n = blockIdx.y;
     const float open = (extra && gate) ? hyb_sigmoid(gate[(size_t)n * ldg]) : 1.f;
     for (int c = blockIdx.x * blockDim.x + threadIdx.x; c < d; c += gridDim.x * blockDim.x) {
         float acc = extra ? open * to_float(extra[(size_t)n * d + c]) : 0.f;
-        for (int r = 0; r < top; ++r)
-            acc = fmaf(weight[(size_t)n * top + r], y[(size_t)place[(size_t)n * top + r] * d + c], acc);
+        for (int r = 0; r < top; ++r) {
+            const int at = place[(size_t)n * top + r];
+            acc = fmaf(weight[(size_t)n * top + r], at >= 0 ? y[(size_t)at * d + c] : to_float(through[(size_t)n * d + c]), acc);
+        }
         out[(size_t)n * d + c] = acc;
     }
 }
 
 SOC_EXPORT int soc_moe_combine(const float* y, const int* place, const float* weight, const void* extra, const float* gate, int ldg,
-                               float* out, int N, int d, int top, int dtype, hipStream_t stream) {
+                               const void* through, float* out, int N, int d, int top, int dtype, hipStream_t stream) {
     if (N <= 0 || d <= 0) return 0;
     if (N > 65535) return (int)hipErrorInvalidValue;
     const dim3 grid((d + 255) / 256 < 16 ? (d + 255) / 256 : 16, N);
     if (dtype == 0)
-        hipLaunchKernelGGL(moe_combine_kernel<float>, grid, dim3(256), 0, stream, y, place, weight, (const float*)extra, gate, ldg, out, N, d, top);
+        hipLaunchKernelGGL(moe_combine_kernel<float>, grid, dim3(256), 0, stream, y, place, weight, (const float*)extra, gate, ldg, (const float*)through, out, N, d, top);
     else
-        hipLaunchKernelGGL(moe_combine_kernel<bf16>, grid, dim3(256), 0, stream, y, place, weight, (const bf16*)extra, gate, ldg, out, N, d, top);
+        hipLaunchKernelGGL(moe_combine_kernel<bf16>, grid, dim3(256), 0, stream, y, place, weight, (const bf16*)extra, gate, ldg, (const bf16*)through, out, N, d, top);
     return soc_last_error();
 }
 

@@ -63,6 +63,8 @@ class ModelRunner:
         self._graph_pool = None          # one memory pool for all captures: replays never overlap
         self.graphs_refused = None       # why enable_graphs left the steps eager, if it did
         self._graph_epoch = 0            # the kernel set's ``graph_epoch`` the held graphs were captured under
+        if getattr(model.plan, "max_positions", None) is not None and cache.max_len > model.plan.max_positions:
+            raise ValueError(f"rows of {cache.max_len} tokens, the model's table of positions holds {model.plan.max_positions}")
         if hasattr(model, "reserve"):
             model.reserve(cache.max_len)     # tables by position stand at their final addresses from here on
         # eager steps: the batch's integers go through pinned staging memory, one copy per step
@@ -79,6 +81,8 @@ class ModelRunner:
             ops = HipKernels(dtype, device)
         weights = load_weights(folder, expected_tensors(plan), dtype, device, plan.duplicates, plan.ignorable)
         model = DecoderModel(plan, weights, ops)
+        if plan.max_positions is not None:
+            max_len = min(max_len, plan.max_positions)      # (no row is longer than the table of positions)
         cache = CacheManager(cache_needs(plan), max_rows=max_rows, max_len=max_len,
                              block_size=block_size, num_blocks=num_blocks, dtype=dtype,
                              device=device)

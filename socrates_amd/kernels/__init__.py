@@ -14,7 +14,8 @@ arithmetic of key splits,
 ``mixers.py`` the mixers with a state per row, attention over a cached latent and blocks with norms
 on both sides of a branch, ``hybrid.py`` attention whose keys and values differ in size, retention, routed
 experts and a per-token side input, ``memory.py`` a matrix memory with exponential gates and the two maps of
-differential attention, ``common.py`` what they share, ``build.py`` the compiler and loader.
+differential attention, ``delta.py`` the gated delta rule, ``streams.py`` several copies of the residual stream,
+``common.py`` what they share, ``build.py`` the compiler and loader.
 """
 
 from __future__ import annotations
@@ -26,6 +27,7 @@ import torch
 
 from .attention import Attention
 from .composite import Composite
+from .delta import Delta
 from .hybrid import Hybrid
 from .latent import Latent
 from .memory import Memory
@@ -35,12 +37,13 @@ from .common import (_ATTENTION_SIGNATURES, _ATTENTION_UP_TO_256, _DTYPE_CODE, _
                      NormOwed, RowsByTile, _check, _declare, _ptr)
 from .planning import MAX_KEY_SPLITS, plan_key_splits
 from .products import Products
+from .streams import Streams
 
 __all__ = ["HipKernels", "KernelBuildError", "KernelError", "MAX_KEY_SPLITS", "NormOwed", "RowsByTile", "build_all",
            "compile_library", "load_library", "plan_key_splits"]
 
 
-class HipKernels(Products, Attention, Latent, Mixers, Hybrid, Composite, Memory):
+class HipKernels(Products, Attention, Latent, Mixers, Hybrid, Composite, Memory, Streams, Delta):
     def __init__(self, dtype=torch.bfloat16, device="cuda:0"):
         if dtype not in _DTYPE_CODE:
             raise ValueError(f"compute dtype must be float32 or bfloat16, not {dtype}")

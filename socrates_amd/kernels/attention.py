@@ -174,8 +174,13 @@ class Attention:
         G = Hq // Hkv
         tokens_per_block = max(1, (16 * rt) >> gpl)
         blocks, n_blocks = self._row_blocks(ctx, N, tokens_per_block, which)
-        split_len, n_splits = self.plan_mfma(n_blocks, Hkv, G, ctx.max_ctx_len)
-        if self.attention_splits is None and n_splits > 1:
+        # (a token of a chunk sees no more keys than its chunk holds, a block of them no more than with the block's own)
+        longest = ctx.max_ctx_len if w >= 0 else min(ctx.max_ctx_len, -w + tokens_per_block)
+        if self.attention_splits is not None or w >= 0:
+            split_len, n_splits = self.plan_mfma(n_blocks, Hkv, G, ctx.max_ctx_len)
+        else:
+            split_len, n_splits = self.plan_mfma(n_blocks, Hkv, G, longest)
+        if self.attention_splits is None and (n_splits > 1 or w < 0):
             split_len = 0           # the kernel shares every row's own keys out evenly among the splits
         part_o = part_ml = None
         if n_splits > 4:
@@ -276,7 +281,8 @@ class Attention:
         (float: scores become softcap * tanh(scores / softcap)), ``sinks`` (float32 [Hq]: one
         more logit per head in the softmax's sum, with no value) and ``slopes`` (float32 [Hq]:
         slope * (key position - query position) added to the scaled scores) and ``keep_first``
-        (int, with a window: the keys at positions below it stay visible to every later token) and ``pooled`` (the
+        (int, with a window: the keys at positions below it stay visible to every later token), ``chunk`` (int c, in
+        place of a window: a token sees the keys of its own chunk of c positions) and ``pooled`` (the
         cache slot, whose pages of means hold one mean key and value per block of ``slot.pool`` positions: a token sees
         the blocks that end before its window begins, in the same softmax). Such a layer,
         and one whose scale is not positive, goes to the kernel that computes scores on the
@@ -296,11 +302,15 @@ class Attention:
         G = Hq // Hkv
         softcap, sinks, slopes, keep_first, means, pool = 0.0, None, None, 0, None, 0
         if terms:
-            known = {"softcap", "sinks", "slopes", "keep_first", "zero_sink", "pooled"}
+            known = {"softcap", "sinks", "slopes", "keep_first", "zero_sink", "pooled", "chunk"}
             if set(terms) - known:
                 raise KernelError(f"attention: unknown score terms {sorted(set(terms) - known)}")
             softcap = float(terms.get("softcap") or 0.0)
-            keep_first = int(terms.get("keep_first") or 0) if w else 0
+            if terms.get("chunk") is not None:
+                if w or terms.get("keep_first") or int(terms["chunk"]) < 1:
+                    raise KernelError("attention: chunks hold at least one position and take the place of a window")
+                w = -int(terms["chunk"])            # (what the kernels know chunks by)
+            keep_first = int(terms.get("keep_first") or 0) if w > 0 else 0
             if keep_first < 0:
                 raise KernelError("attention: the number of first keys that stay visible is not negative")
             sinks, slopes = terms.get("sinks"), terms.get("slopes")
@@ -312,7 +322,7 @@ class Attention:
             if terms.get("pooled") is not None:
                 # the slot itself: its pages of means and how many positions a mean stands for
                 means, pool = terms["pooled"].pooled, int(terms["pooled"].pool)
-                if means is None or pool < 1 or not w or keep_first or slopes is not None:
+                if means is None or pool < 1 or w <= 0 or keep_first or slopes is not None:
                     raise KernelError("attention: pooled blocks need a window, the slot's pages of means, and neither kept "
                                       "first keys nor a bias by distance")
                 self._check_slot(means, Hkv, D)
@@ -403,7 +413,7 @@ class Attention:
                 self._wave_attention(lib, q, slot, ctx, out, scale, w, rt, gpl, None, softcap)
                 return out
         self.last_attention_kernel = ("tokens", 0)
-        max_keys = ctx.max_ctx_len if not w else min(w + keep_first, ctx.max_ctx_len)
+        max_keys = ctx.max_ctx_len if not w else min(abs(w) + keep_first, ctx.max_ctx_len)
         if pool:
             max_keys = min(w, ctx.max_ctx_len) + max(0, ctx.max_ctx_len - w) // pool
         split_len, n_splits = self.plan_splits(N, Hkv, G, max_keys)

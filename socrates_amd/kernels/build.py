@@ -42,7 +42,8 @@ LATENT_VGPR_MAX_WIDTH = 256
 
 SOURCES = {"elementwise": "elementwise.hip", "gemm": "gemm.hip", "sampling": "sampling.hip",
            "attention": "attention.hip", "mixers": "mixers.hip", "hybrid": "hybrid.hip",
-           "composite": "composite.hip", "memory": "memory.hip", "latent": "latent.hip"}
+           "composite": "composite.hip", "memory": "memory.hip", "latent": "latent.hip",
+           "streams": "streams.hip", "delta": "delta.hip"}
 # head sizes built ahead by build_all(): the common ones and those the tests use, so that
 # no test compiles on the GPU box
 COMMON_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 112, 128, 160, 256, 272, 288, 512, 576)

@@ -71,10 +71,10 @@ _HYBRID_SIGNATURES = {
     "soc_head_gate": [P, P, I, P, I, I, I, I, I, P],
     "soc_retention": [P, I, I, I, I, P, P, I, F, P, I, I, I, P, L, I, P, P, P, I, P, I, I, I, P],
     "soc_relu_squared": [P, P, L, I, P],
-    "soc_moe_route": [P, I, P, P, I, I, I, I, I, F, I, I, F, P, P, P],
+    "soc_moe_route": [P, I, P, P, I, I, I, I, I, F, I, I, F, I, P, P, P],
     "soc_moe_sort": [P, I, I, I, I, P, P, P, P, P],
     "soc_grouped_linear": [P, I, P, I, P, P, P, I, I, P, I, I, I, F, F, F, I, I, I, P],
-    "soc_moe_combine": [P, P, P, P, P, I, P, I, I, I, I, P],
+    "soc_moe_combine": [P, P, P, P, P, I, P, P, I, I, I, I, P],
     "soc_side_gate": [P, P, I, I, P, I, P, I, I, I, P],
     "soc_add_cast": [P, P, P, I, L, P, I, P],
 }
@@ -93,6 +93,14 @@ _MEMORY_SIGNATURES = {
     "soc_memory_gates": [P, P, F, P, I, I, I, F, I, I, P, L, I, P, P, I, I, I, P, P, P, P, I, P],
     "soc_memory_finish": [P, P, P, I, P, I, I, I, F, F, P, I, P],
     "soc_diff_combine": [P, P, I, I, I, I, I, F, F, F, I, P],
+}
+_STREAMS_SIGNATURES = {
+    "soc_embedding_streams": [P, P, F, P, P, I, P, I, I, I, I, I, P],
+    "soc_streams": [P, I] + [P, I, P, P, I, P, F] * 2 + [P, P, P, P, P, F, I, P, P, I, I, I, I, P],
+}
+_DELTA_SIGNATURES = {
+    "soc_delta_prepare": [P] + [I] * 7 + [P, I, F, F, P, P, P, P, L, I, P, P, P, P, P, I, I, I, P],
+    "soc_delta_walk": [P, P, P, I, I, I, I, I, P, L, I, P, P, P, I, I, P],
 }
 _SAMPLING_SIGNATURES = {"soc_sample": [P, P, P, P, P, I, I, P], "soc_argmax": [P, P, P, I, I, I, P]}
 _ATTENTION_SIGNATURES = {

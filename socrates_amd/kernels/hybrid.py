@@ -31,11 +31,12 @@ class ExpertRuns:
 
 class ExpertSums:
     """What the experts of a step have left, before a token's weighted sum is taken: ``y`` float32 [M, d] by place,
-    ``runs`` (where each (token, choice) pair lies) and ``weight`` [N, top]. Taken by ``branches_add``."""
-    __slots__ = ("y", "runs", "weight")
+    ``runs`` (where each (token, choice) pair lies) and ``weight`` [N, top]; ``through`` (compute dtype [N, d] or None):
+    what a pair without a place stands for, the experts' input. Taken by ``branches_add`` and ``streams_update``."""
+    __slots__ = ("y", "runs", "weight", "through")
 
-    def __init__(self, y, runs, weight):
-        self.y, self.runs, self.weight = y, runs, weight
+    def __init__(self, y, runs, weight, through=None):
+        self.y, self.runs, self.weight, self.through = y, runs, weight, through
 
 
 class Hybrid:
@@ -158,13 +159,13 @@ class Hybrid:
     _SCORING = {"softmax": 0, "sigmoid": 1, "chosen": 2}
 
     def moe_route(self, logits, correction, top, n_groups=1, keep_groups=1, renorm_eps=1e-20, scoring="softmax", group_top=1,
-                  scale=1.0, bias=None):
+                  scale=1.0, bias=None, renorm=True):
         """logits float32 [N, E] (they may be columns of a wider product): scores are their softmax, or with ``scoring``
         "sigmoid" the sigmoid of each, or with "chosen" the weights are the softmax over the chosen logits and the choice
         goes by the logits themselves; ``bias`` (float32 [E]) is added to the logits first. The choice goes by score + correction among the experts of the ``keep_groups``
         best of ``n_groups`` equal groups of neighbours (a group's score is the sum of its ``group_top`` best choice
         scores). Returns (experts int32 [N, top], weights float32 [N, top]: the chosen scores over their sum, times
-        ``scale``)."""
+        ``scale``; ``renorm`` False: as they are, times ``scale``)."""
         N, E = logits.shape
         if (logits.device.type != "cuda" or logits.dtype != torch.float32 or logits.stride(1) != 1
                 or (N > 1 and logits.stride(0) < E)):
@@ -182,14 +183,14 @@ class Hybrid:
         weight = torch.empty((N, top), dtype=torch.float32, device=self.device)
         _check(self._hybrid().soc_moe_route(_ptr(logits), c_int(logits.stride(0) if N > 1 else E), _ptr(bias), _ptr(correction), c_int(N), c_int(E),
                                             c_int(top), c_int(n_groups), c_int(keep_groups), c_float(renorm_eps),
-                                            c_int(self._SCORING[scoring]), c_int(group_top), c_float(scale), _ptr(idx),
+                                            c_int(self._SCORING[scoring]), c_int(group_top), c_float(scale), c_int(1 if renorm else 0), _ptr(idx),
                                             _ptr(weight), self._stream()),
                "moe_route")
         return idx, weight
 
     def moe_sort(self, idx, E, tile=EXPERT_TILE):
         """The (token, choice) pairs of ``idx`` [N, top] laid out expert by expert, in tiles of ``tile`` places: an
-        ``ExpertRuns``."""
+        ``ExpertRuns``. A pair of an expert from E on has no place (-1)."""
         N, top = idx.shape
         self._want(idx, "experts", torch.int32)
         if not 1 <= E <= MAX_EXPERTS:
@@ -236,16 +237,18 @@ class Hybrid:
             self._stream()), "grouped_linear")
         return out
 
-    def moe_combine(self, y, runs, weight, extra=None, extra_gate=None):
+    def moe_combine(self, y, runs, weight, extra=None, extra_gate=None, through=None):
         """float32 [N, d]: each token's weighted sum of its experts' rows of ``y`` (float32 [M, d] by place), plus
         ``extra`` [N, d] (compute dtype) if given, times sigmoid(``extra_gate``) (float32 [N], which may be a column
-        of a wider product) if that is given."""
+        of a wider product) if that is given. A pair without a place stands for the token's row of ``through`` [N, d]."""
         N, top = weight.shape
         d = y.shape[1]
         self._want(y, "expert results", torch.float32, (N * top, d))
         self._want(weight, "weights", torch.float32)
         if extra is not None:
             self._want(extra, "extra", self.dtype, (N, d))
+        if through is not None:
+            self._want(through, "the experts' input", self.dtype, (N, d))
         ldg = 0
         if extra_gate is not None:
             if (extra is None or extra_gate.device.type != "cuda" or extra_gate.dtype != torch.float32
@@ -259,7 +262,7 @@ class Hybrid:
             _check(self._hybrid().soc_moe_combine(_ptr(y), _ptr(runs.place[lo * top:]), _ptr(weight[lo:]),
                                                   _ptr(extra[lo:]) if extra is not None else None,
                                                   _ptr(extra_gate[lo:]) if extra_gate is not None else None, c_int(ldg),
-                                                  _ptr(out[lo:]), c_int(n), c_int(d),
+                                                  _ptr(through[lo:]) if through is not None else None, _ptr(out[lo:]), c_int(n), c_int(d),
                                                   c_int(top), c_int(self.code), self._stream()), "moe_combine")
         return out
 
@@ -271,26 +274,33 @@ class Hybrid:
             return next((t for least, t in EXPERT_TILES_MANY if M >= least * E), EXPERT_TILE)
         return EXPERT_TILE
 
-    def moe_experts(self, x, idx, weight, w_gate_up, w_down, limit, slope, extra=None, shift=1.0, extra_gate=None):
+    def moe_experts(self, x, idx, weight, w_gate_up, w_down, limit, slope, extra=None, shift=1.0, extra_gate=None, whole=True,
+                    identity=False):
         """The weighted sum of each token's chosen experts (gated feed-forwards with the activation
         g sigmoid(slope g) (u + shift) under a clamp: ``w_gate_up`` [E, 2 ff, d], ``w_down`` [E, d, ff]) plus ``extra``
-        (times sigmoid(``extra_gate``) per token if given); float32 [N, d]."""
+        (times sigmoid(``extra_gate``) per token if given); float32 [N, d]. ``identity``: choices from E on are identity
+        experts, whose result is x. ``whole`` False (without an extra term): an ``ExpertSums``, the weighted sum left to
+        the caller's own sum."""
         E, _, d = w_gate_up.shape
         runs = self.moe_sort(idx, E, self._expert_tile(x, idx.numel(), E, d, w_down.shape[2]))
         act = self.grouped_linear(x, w_gate_up, runs, by_token=True, glu=(limit, slope, shift))
         y = self.grouped_linear(act, w_down, runs, by_token=False, out_dtype=torch.float32)
-        return self.moe_combine(y, runs, weight, extra, extra_gate)
+        through = x if identity else None
+        if not whole and extra is None:
+            return ExpertSums(y, runs, weight, through)
+        return self.moe_combine(y, runs, weight, extra, extra_gate, through)
 
-    def moe_experts_squared(self, x, idx, weight, w_up, w_down, extra=None, extra_gate=None, whole=True):
+    def moe_experts_squared(self, x, idx, weight, w_up, w_down, extra=None, extra_gate=None, whole=True, identity=False):
         """The same with experts Wd relu(Wu x)^2 (``w_up`` [E, ff, d], ``w_down`` [E, d, ff]). ``whole`` False (without
         an extra term): an ``ExpertSums``, the weighted sum left to ``branches_add``."""
         E, ff, d = w_up.shape
         runs = self.moe_sort(idx, E, self._expert_tile(x, idx.numel(), E, d, ff))
         act = self.grouped_linear(x, w_up, runs, by_token=True, squared=True)
         y = self.grouped_linear(act, w_down, runs, by_token=False, out_dtype=torch.float32)
+        through = x if identity else None
         if not whole and extra is None:
-            return ExpertSums(y, runs, weight)
-        return self.moe_combine(y, runs, weight, extra, extra_gate)
+            return ExpertSums(y, runs, weight, through)
+        return self.moe_combine(y, runs, weight, extra, extra_gate, through)
 
     # -- a per-token side input, and the residual sum with a cast -----------------------------------------------------
     def side_gate(self, t, table, col0, token_ids):

@@ -66,6 +66,8 @@ class Mixers:
             if scale is not None:
                 self._want(scale, "branch scale", torch.float32, (d,))
             if isinstance(y, ExpertSums):
+                if y.through is not None:
+                    raise KernelError("branches_add: no identity experts")
                 top = y.weight.shape[1]
                 self._want(y.y, "expert results", torch.float32, (N * top, d))
                 self._want(y.weight, "expert weights", torch.float32, (N, top))
@@ -203,15 +205,15 @@ class Mixers:
     def gated_group_norm(self, y, z, gain, groups, eps, gate_first=True, sigmoid=False):
         """y (float32 [N, inner]) * silu(z[:, :inner]), RMS-normed in ``groups`` equal parts, times gain;
         ``gate_first`` False: y normed, times gain, and only then times silu(z). ``sigmoid``: the gate is
-        sigmoid(z) in place of silu(z)."""
+        sigmoid(z) in place of silu(z). ``z`` may be columns of a wider product."""
         N, inner = y.shape
         self._want(y, "y", torch.float32)
-        self._want(z, "z", self.dtype)
         self._want(gain, "gain", torch.float32, (inner,))
-        if z.dim() != 2 or z.shape[0] != N or z.shape[1] < inner or groups < 1 or inner % groups:
+        if (z.device.type != "cuda" or z.dtype != self.dtype or z.dim() != 2 or z.shape[0] != N or z.shape[1] < inner
+                or z.stride(1) != 1 or (N > 1 and z.stride(0) < z.shape[1]) or groups < 1 or inner % groups):
             raise KernelError(f"gated norm: z {tuple(z.shape)} against y {tuple(y.shape)} in {groups} parts")
         out = torch.empty((N, inner), dtype=self.dtype, device=self.device)
-        _check(self._mixers().soc_gated_group_norm(_ptr(y), _ptr(z), c_int(z.shape[1]), _ptr(gain), c_int(N), c_int(inner),
+        _check(self._mixers().soc_gated_group_norm(_ptr(y), _ptr(z), c_int(z.stride(0) if N > 1 else z.shape[1]), _ptr(gain), c_int(N), c_int(inner),
                                                    c_int(groups), c_float(eps), c_int(1 if gate_first else 0), c_int(1 if sigmoid else 0),
                                                    _ptr(out),
                                                    c_int(self.code), self._stream()),

@@ -1,4 +1,4 @@
-from . import (attention, block, differential_attention, feedforward, gated_attention, latent_attention,  # noqa: F401
+from . import (attention, block, delta, differential_attention, feedforward, gated_attention, latent_attention,  # noqa: F401
                linear_attention, matrix_memory, norm, parallel, recurrent, retention, rope, routed, side, window_attention)  # noqa: F401  (registers the parts)
 from .block import build_block, register_arrangement
 from .model import DecoderModel, cache_needs, expected_tensors

@@ -8,7 +8,7 @@ branch output un-added ("pending") and the next norm adds it.
 
 from __future__ import annotations
 
-from ..config.specs import BlockSpec, DepthAverageSpec, LayerScaleSpec
+from ..config.specs import BlockSpec, DepthAverageSpec, LayerScaleSpec, StreamsSpec
 from .registry import TensorDecl, build_part, register_part, tensors_of
 
 _ARRANGEMENTS = {}
@@ -349,11 +349,71 @@ class ParallelBlock:
         return None if rows is None else Normed(rows)
 
 
+class Streams:
+    """Holds how a branch reads and writes the copies of the stream; the block applies it where it adds a branch up."""
+
+    @staticmethod
+    def tensors(spec: StreamsSpec):
+        return {"in": TensorDecl((spec.n,), "vector"), "mix": TensorDecl((spec.n, spec.n), "vector"), "out": TensorDecl((spec.n,), "vector")}
+
+    def __init__(self, spec: StreamsSpec, tensors, ops):
+        self.spec = spec
+        self.read, self.mix, self.out = (tensors[k].contiguous() for k in ("in", "mix", "out"))
+
+
+class StreamsBlock:
+    """Several copies x_1 .. x_s of the stream, float32 [N, s, d]: a branch reads u = sum_a in[a] x_a through its norm,
+    and with y its result x_b <- sum_a mix[a, b] x_a + out[b] y, all b at once; first the mixer, then the feed-forward
+    (a layer may have none). One kernel closes a branch: it adds up the branch's results (two scaled ones, partial sums,
+    or the experts' results by place), takes the new copies from the old ones, and reads and norms what the next branch
+    works on, which may be the next block's first."""
+    chains = True
+    # (as for the sandwich: the library's tuning pass is kept to the models it was measured with)
+    library_tuning = False
+
+    def __init__(self, spec: BlockSpec, weights, ops):
+        self.spec, self.ops = spec, ops
+        for role in ("norm1", "mixer", "norm2", "ffn", "streams1", "streams2"):
+            sub = getattr(spec, role)
+            setattr(self, role, None if sub is None else build_part(sub, _sub_tensors(spec, role, weights), ops))
+        if self.streams1 is None or (self.ffn is not None and (self.norm2 is None or self.streams2 is None)):
+            raise ValueError("every branch needs its norm and how it reads and writes the copies of the stream")
+        parts = (self.norm1, self.mixer, self.norm2, self.ffn)
+        self.capturable = all(getattr(p, "capturable", True) for p in parts if p is not None)
+
+    def reserve(self, n_positions):
+        for part in (self.mixer, self.ffn):
+            if hasattr(part, "reserve"):
+                part.reserve(n_positions)
+
+    def _close(self, residual, y, streams, follows):
+        """``follows``: (how the next branch reads the copies, its norm's terms), or None: the copies only."""
+        branches = y if isinstance(y, list) else [(y, 1.0)]
+        read, norm = follows if follows is not None else (None, None)
+        return self.ops.streams_update(residual, branches, streams.mix, streams.out, read, norm)
+
+    def forward(self, residual, pending, ctx, slot, write=True, nxt=None):
+        ops = self.ops
+        h = pending.rows if isinstance(pending, Normed) else ops.streams_norm(residual, self.streams1.read, self.norm1.terms())
+        apart = {"apart": True} if getattr(self.mixer, "offers_branches", False) else {}
+        y = self.mixer.forward(h, ctx, slot, write, **apart)
+        then = (nxt.streams1.read, nxt.norm1.terms()) if isinstance(nxt, StreamsBlock) else None
+        if self.ffn is not None:
+            h = self._close(residual, y, self.streams1, (self.streams2.read, self.norm2.terms()))
+            sums = {"whole": False} if getattr(self.ffn, "offers_sums", False) else {}
+            h = self._close(residual, self.ffn.forward(h, ctx, **sums), self.streams2, then)
+        else:
+            h = self._close(residual, y, self.streams1, then)
+        return None if h is None else Normed(h)
+
+
 register_arrangement("parallel_scaled", ParallelBlock)
 register_arrangement("postnorm_depth", DepthAverageBlock)
 register_arrangement("prenorm", PreNormBlock)
 register_arrangement("prenorm_side", SideInputBlock)
 register_arrangement("sandwich", SandwichBlock)
+register_arrangement("streams", StreamsBlock)
 
 register_part(DepthAverageSpec, DepthAverage)
 register_part(LayerScaleSpec, LayerScale)
+register_part(StreamsSpec, Streams)

@@ -24,6 +24,8 @@ def expected_tensors(plan: ModelPlan):
         out[_joined(plan.final_norm_prefix, local)] = decl
     if plan.head_name is not None:
         out[plan.head_name] = TensorDecl((plan.vocab_size, plan.hidden))
+    if plan.positions_name is not None:
+        out[plan.positions_name] = TensorDecl((plan.max_positions, plan.hidden))
     return out
 
 
@@ -52,6 +54,7 @@ class DecoderModel:
                         for local in tensors_of(plan.final_norm)}
         self.final_norm = build_part(plan.final_norm, norm_tensors, ops)
         self.head = self.embed if plan.head_name is None else weights[plan.head_name]
+        self.position_table = weights[plan.positions_name] if plan.positions_name is not None else None
         # False if any part declares `capturable = False`: the runner then captures the runs of
         # blocks between such parts and runs those as they come (``segments``); a final norm
         # that cannot be captured leaves every step eager
@@ -76,8 +79,13 @@ class DecoderModel:
     # The forward pass in pieces, for a runner that captures what can be captured and runs
     # the rest as it comes: begin (the embedding), run (some entries of the run order), finish
     # (final norm and head). ``residual`` is one float32 tensor from begin to finish, updated
-    # in place; ``pending`` is what the last block left un-added.
+    # in place ([tokens, hidden], or [tokens, copies, hidden] where the plan has copies of the
+    # stream); ``pending`` is what the last block left un-added.
     def begin(self, ctx):
+        if self.position_table is not None or self.plan.streams is not None:
+            x = self.ops.embedding_streams(ctx.token_ids, self.embed, self.plan.embedding_scale, ctx.positions,
+                                           self.position_table, self.plan.streams or 1)
+            return (x if self.plan.streams is not None else x.view(-1, self.plan.hidden)), None
         residual = self.ops.embedding(ctx.token_ids, self.embed)
         if self.plan.embedding_scale != 1.0:
             self.ops.scale_softcap_(residual, self.plan.embedding_scale)
@@ -105,6 +113,11 @@ class DecoderModel:
         if ctx.n_want == 0:
             # The cache is complete after the last block; no logits are asked for.
             return torch.empty((0, self.plan.vocab_size), dtype=torch.float32, device=self.ops.device)
+        if self.plan.streams is not None:
+            # (blocks leave nothing un-added in the copies of the stream; what is normed is their sum)
+            if pending is not None:
+                raise ValueError("a block left something un-added to the copies of the stream")
+            return self.head_logits(self.ops.streams_norm(residual, None, self.final_norm.terms(), ctx.want_index))
         # (the normed rows go to the head's product and nowhere else: their layout is the kernel set's)
         if getattr(self.final_norm, "free_layout", False):
             h = self.final_norm.add_norm(residual, pending, rows=ctx.want_index, by_tile=True)

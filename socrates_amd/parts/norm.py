@@ -2,13 +2,14 @@
 
 eps sits inside the square root and the gain is the plain weight, as in the
 reference. Statistics are taken in float32 whatever the compute dtype.
+``LayerNorm`` takes the mean off first and adds a bias.
 """
 
 from __future__ import annotations
 
 import torch
 
-from ..config.specs import RMSNormSpec, ScalarRMSNormSpec
+from ..config.specs import LayerNormSpec, RMSNormSpec, ScalarRMSNormSpec
 from .registry import TensorDecl, register_part
 
 
@@ -40,6 +41,10 @@ class RMSNorm:
         around it (``HipKernels.linear_add_norm``)."""
         return self.weight, self.spec.eps
 
+    def terms(self):
+        """(gain, bias or None, eps, whether the mean is taken off): what the kernel for copies of the stream needs."""
+        return self.weight, None, self.spec.eps, False
+
     def __call__(self, x):
         """Plain norm over the last dimension of ``x`` (any leading shape)."""
         return self.ops.rmsnorm(x, self.weight, self.spec.eps)
@@ -58,5 +63,34 @@ class ScalarRMSNorm(RMSNorm):
         self.weight = tensors[""].to(torch.float32).reshape(1).expand(spec.dim).contiguous()
 
 
+class LayerNorm:
+    """y = (x - mean) / sqrt(variance + eps) * w + b, the variance being the mean of the squared deviations."""
+
+    @staticmethod
+    def tensors(spec: LayerNormSpec):
+        return {"": TensorDecl((spec.dim,), "vector"), "b": TensorDecl((spec.dim,), "vector")}
+
+    def __init__(self, spec: LayerNormSpec, tensors, ops):
+        self.spec, self.ops = spec, ops
+        self.weight, self.bias = (tensors[k].to(torch.float32).contiguous() for k in ("", "b"))
+
+    def terms(self):
+        return self.weight, self.bias, self.spec.eps, True
+
+    def add_norm(self, residual, delta, rows=None):
+        """As ``RMSNorm.add_norm``; with ``rows`` and a ``delta`` only the rows' sum is taken, and the stream is left
+        as it is."""
+        N, d = residual.shape
+        if delta is not None and rows is not None:
+            residual = residual[rows.long()].contiguous()
+            delta = delta.index_select(delta.dim() - 2, rows.long()).contiguous()
+            rows = None
+        view = residual.view(residual.shape[0], 1, d)
+        if delta is None:
+            return self.ops.streams_norm(view, None, self.terms(), rows)
+        return self.ops.streams_update(view, [(delta, 1.0)], None, None, None, self.terms())
+
+
 register_part(RMSNormSpec, RMSNorm)
+register_part(LayerNormSpec, LayerNorm)
 register_part(ScalarRMSNormSpec, ScalarRMSNorm)

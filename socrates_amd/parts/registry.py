@@ -68,12 +68,16 @@ class PagedKV:
     their own (entry b of a row stands for positions bP .. bP + P - 1), and a token's page is held until the
     block of its last position is complete, so that the means can be taken from the pages.
 
+    ``chunk`` = c, in place of a window: a token sees the positions of its own chunk of c positions (counted from 0), so
+    a page all of whose positions lie in earlier chunks is given back.
+
     A mixer made of several mixers names a tuple of needs; its slot is then the tuple of their slots."""
     n_kv_heads: int
     head_dim: int
     window: Optional[int] = None
     keep_first: int = 0
     pool: int = 0
+    chunk: Optional[int] = None
 
 
 @dataclass(frozen=True)

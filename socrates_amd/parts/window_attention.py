@@ -2,8 +2,8 @@
 the projections, an RMS norm of q and k per head or over the whole projection, a rotation over
 interleaved pairs with stretched frequencies, values turned by their position and the result turned
 back, one mean key and value per block of tokens that lies before the window, a learned sink per head,
-kept first keys, a soft cap on the scores, a norm of q and k behind the rotation, values that are the
-keys as projected, and a sigmoid gate per head.
+kept first keys, chunks of positions in place of the window, a soft cap on the scores, a norm of q and k
+behind the rotation, values that are the keys as projected, and a sigmoid gate per head.
 
 One product reads the layer's input: rows [q | k | v]. One kernel adds the biases, norms and turns q
 and k, turns the values and writes keys and values to the token's place in the pages; both pools have
@@ -60,7 +60,7 @@ class WindowAttention:
     @staticmethod
     def cache_need(spec: WindowAttentionSpec):
         return PagedKV(spec.n_kv_heads, spec.cache_width, spec.window, spec.keep_first if spec.window is not None else 0,
-                       spec.pool)
+                       spec.pool, spec.chunk)
 
     def __init__(self, spec: WindowAttentionSpec, tensors, ops):
         self.spec, self.ops = spec, ops
@@ -88,16 +88,20 @@ class WindowAttention:
         self.magnitude = spec.position.magnitude if spec.position is not None else 1.0
         if spec.head_gate and spec.value_base is not None:
             raise ValueError("a gate per head and values turned back are not combined here")
+        # a caller may take the first product with other rows (the bias then does not fit its columns)
+        self.takes_first = self.bias is None
 
-    def forward(self, x, ctx, slot, write=True, out_dtype=None, raw=False):
-        """``raw``: return (product, the output projection's bias or None) and leave the bias to the caller."""
+    def forward(self, x, ctx, slot, write=True, out_dtype=None, raw=False, first=None):
+        """``raw``: return (product, the output projection's bias or None) and leave the bias to the caller. ``first`` =
+        (rows, column): ``w_first``'s product is in these rows from that column on, the caller has taken it."""
         s, ops = self.spec, self.ops
         H, G, D, Dv, P = s.n_heads, s.n_kv_heads, s.head_dim, s.v_dim, s.cache_width
         if not write:
             raise ValueError("this attention writes the cache slot it reads")
-        first = ops.linear(x, self.w_first)
+        first, at = first if first is not None else (ops.linear(x, self.w_first), 0)
+        cols = tuple(at + c for c in self.cols)
         more = {} if self.magnitude == 1.0 else {"magnitude": self.magnitude}
-        q = ops.window_prepare(first, self.cols, H, G, D, Dv, P, self.bias, self.q_gain, self.k_gain, s.qk_norm, s.eps,
+        q = ops.window_prepare(first, cols, H, G, D, Dv, P, self.bias, self.q_gain, self.k_gain, s.qk_norm, s.eps,
                                self.inv_freq, self.rotary_dim, self.value_freq, ctx.positions, ctx.token_rows, slot, **more)
         terms = {}
         if self.sinks is not None:
@@ -106,12 +110,14 @@ class WindowAttention:
             terms["softcap"] = s.softcap
         if s.window is not None and s.keep_first:
             terms["keep_first"] = s.keep_first
+        if s.chunk is not None:
+            terms["chunk"] = s.chunk
         if s.pool:
             ops.pool_blocks(slot, ctx)
             terms["pooled"] = slot
         o = ops.paged_attention(q, slot, ctx, s.scale, s.window, terms=terms or None)
         if s.head_gate:
-            o = ops.head_gate(o, H, P, Dv, first[:, self.col_gate:self.col_gate + H])
+            o = ops.head_gate(o, H, P, Dv, first[:, at + self.col_gate:at + self.col_gate + H])
         elif self.value_freq is not None or P != Dv:
             o = ops.turn_back(o, H, P, Dv, self.value_freq, ctx.positions)
         y = ops.linear(o, self.w_o, out_dtype=out_dtype)

@@ -129,7 +129,7 @@ class TorchKernels:
         """Token by token: gather the row's keys 0..p through the table, mask the window.
         ``terms``: a bias by distance (``slopes`` [Hq]), a soft cap of the scores, one more
         logit per head in the softmax's sum (``sinks`` [Hq]), first keys that stay visible
-        behind a window (``keep_first``)."""
+        behind a window (``keep_first``), the keys of the token's own chunk only (``chunk``)."""
         terms = terms or {}
         N, Hq, D = q.shape
         Hkv, bs = slot.k.shape[1], slot.block_size
@@ -141,6 +141,8 @@ class TorchKernels:
         for t in range(N):
             p, row = int(positions[t]), int(rows[t])
             lo = 0 if window is None else max(0, p - window + 1)
+            if terms.get("chunk"):
+                lo = p // terms["chunk"] * terms["chunk"]
             idx = np.arange(lo, p + 1)
             if window is not None and terms.get("keep_first"):
                 idx = np.concatenate([np.arange(0, min(int(terms["keep_first"]), lo)), idx])
@@ -408,7 +410,7 @@ class TorchKernels:
         return (torch.relu(x.to(self.acc)) ** 2).to(self.dtype)
 
     def moe_route(self, logits, correction, top, n_groups=1, keep_groups=1, renorm_eps=1e-20, scoring="softmax",
-                  group_top=1, scale=1.0, bias=None):
+                  group_top=1, scale=1.0, bias=None, renorm=True):
         A = self.acc
         z = logits.to(A) if bias is None else logits.to(A) + bias.to(A)
         s = torch.sigmoid(z) if scoring == "sigmoid" else torch.softmax(z, dim=-1)
@@ -433,10 +435,11 @@ class TorchKernels:
             idx[:, r] = first
             taken[torch.arange(N), first] = True
         w = torch.gather(s, 1, idx) if scoring != "chosen" else torch.softmax(torch.gather(z, 1, idx), dim=-1)
-        w = w / (w.sum(-1, keepdim=True) + renorm_eps) * scale
+        w = (w / (w.sum(-1, keepdim=True) + renorm_eps) if renorm else w) * scale
         return idx.to(torch.int32), w.to(torch.float32 if A == torch.float32 else A)
 
-    def moe_experts(self, x, idx, weight, w_gate_up, w_down, limit, slope, extra=None, shift=1.0, extra_gate=None):
+    def moe_experts(self, x, idx, weight, w_gate_up, w_down, limit, slope, extra=None, shift=1.0, extra_gate=None, whole=True,
+                    identity=False):
         A = self.acc
         N, top = idx.shape
         ff = w_gate_up.shape[1] // 2
@@ -445,21 +448,28 @@ class TorchKernels:
             out += extra.to(A) if extra_gate is None else extra.to(A) * torch.sigmoid(extra_gate.to(A)).unsqueeze(-1)
         for r in range(top):
             e = idx[:, r].long()
+            same = e >= w_gate_up.shape[0]
+            e = e.clamp(max=w_gate_up.shape[0] - 1)
             both = torch.einsum("nk,nok->no", x.to(A), w_gate_up[e].to(A)).to(self.dtype)
             act = self.glu_clamped(both, limit, slope, ff, shift)
             y = torch.einsum("nk,nok->no", act.to(A), w_down[e].to(A))
+            y = torch.where(same.unsqueeze(-1), x.to(A), y)
+            assert identity or not bool(same.any())
             out += weight[:, r:r + 1].to(A) * y
         return out.to(torch.float32 if A == torch.float32 else A)
 
-    def moe_experts_squared(self, x, idx, weight, w_up, w_down, extra=None, extra_gate=None, whole=True):
+    def moe_experts_squared(self, x, idx, weight, w_up, w_down, extra=None, extra_gate=None, whole=True, identity=False):
         A = self.acc
         out = torch.zeros((idx.shape[0], w_down.shape[1]), dtype=A, device=x.device)
         if extra is not None:
             out += extra.to(A) if extra_gate is None else extra.to(A) * torch.sigmoid(extra_gate.to(A)).unsqueeze(-1)
         for r in range(idx.shape[1]):
             e = idx[:, r].long()
+            same = e >= w_up.shape[0]
+            e = e.clamp(max=w_up.shape[0] - 1)
             act = (torch.relu(torch.einsum("nk,nok->no", x.to(A), w_up[e].to(A))) ** 2).to(self.dtype)
-            out += weight[:, r:r + 1].to(A) * torch.einsum("nk,nok->no", act.to(A), w_down[e].to(A))
+            assert identity or not bool(same.any())
+            out += weight[:, r:r + 1].to(A) * torch.where(same.unsqueeze(-1), x.to(A), torch.einsum("nk,nok->no", act.to(A), w_down[e].to(A)))
         return out.to(torch.float32 if A == torch.float32 else A)
 
     def side_gate(self, t, table, col0, token_ids):
@@ -630,6 +640,64 @@ class TorchKernels:
         return (g * gate_up[..., ff:2 * ff].to(self.acc)).to(self.dtype)
 
     # -- sampling ----------------------------------------------------------------------------
+    # -- copies of the residual stream -----------------------------------------------------------
+    def embedding_streams(self, ids, table, scale, positions, position_table, n):
+        A = torch.float32 if self.acc == torch.float32 else self.acc
+        x = table[ids.long()].to(A) * scale
+        if position_table is not None:
+            x = x + position_table[positions.long()].to(A)
+        return x.unsqueeze(1).repeat(1, n, 1)
+
+    def streams_norm(self, x, read, norm, rows=None):
+        gain, bias, eps, centred = norm
+        x = x.to(self.acc) if rows is None else x[rows.long()].to(self.acc)
+        u = x.sum(1) if read is None else torch.einsum("s,nsd->nd", read.to(self.acc), x)
+        if centred:
+            u = u - u.mean(-1, keepdim=True)
+        y = self._norm(u, gain, eps)
+        return (y if bias is None else y + bias.to(self.acc)).to(self.dtype)
+
+    def streams_update(self, x, branches, mix, out, read=None, norm=None):
+        old, y = x.to(self.acc), 0.0
+        for b, scale in branches:
+            y = y + scale * (b.sum(0) if b.dim() == 3 else b).to(self.acc)
+        if mix is None:
+            x.copy_(old + y.unsqueeze(1))
+        else:
+            x.copy_(torch.einsum("st,nsd->ntd", mix.to(self.acc), old) + out.to(self.acc).view(1, -1, 1) * y.unsqueeze(1))
+        return None if norm is None else self.streams_norm(x, read, norm)
+
+    # -- gated delta rule ------------------------------------------------------------------------
+    def delta_rule(self, x, col, G, H, D, Dv, taps_w, q_scale, unit_eps, z, a_log, dt_bias, state, conv_offset, offset, ctx):
+        A = self.acc
+        C, back = 2 * G * D + H * Dv, taps_w.shape[1] - 1
+        N = x.shape[0]
+        out = torch.empty((N, H * Dv), dtype=A, device=x.device)
+        beta = torch.sigmoid(z[:, :H].to(A))
+        step = torch.nn.functional.softplus(z[:, H:].to(A) + dt_bias.to(A), threshold=1e9)
+        g = torch.exp(-torch.exp(a_log.to(A)) * step)
+        for row, lo, hi in self._sequences(ctx):
+            kept = state[row, conv_offset:conv_offset + back * C].view(back, C)
+            seen = torch.cat([kept.to(A), x[lo:hi, col:col + C].to(A)])
+            y = sum(seen[j:j + hi - lo] * taps_w[:, j].to(A) for j in range(back + 1))
+            y = y * torch.sigmoid(y)
+            if back:
+                kept.copy_(seen[-back:])
+            q, k = y[:, :G * D].view(-1, G, D), y[:, G * D:2 * G * D].view(-1, G, D)
+            v = y[:, 2 * G * D:].to(self.dtype).to(A).view(-1, H, Dv)
+            q = q / torch.sqrt(q.pow(2).sum(-1, keepdim=True) + unit_eps) * q_scale
+            k = k / torch.sqrt(k.pow(2).sum(-1, keepdim=True) + unit_eps)
+            q, k = q.repeat_interleave(H // G, dim=1), k.repeat_interleave(H // G, dim=1)
+            own = state[row, offset:offset + H * Dv * D].view(H, Dv, D)
+            S = own.to(A)
+            for t in range(hi - lo):
+                S = S * g[lo + t].view(H, 1, 1)
+                u = beta[lo + t].unsqueeze(-1) * (v[t] - torch.einsum("hvk,hk->hv", S, k[t]))
+                S = S + u.unsqueeze(-1) * k[t].unsqueeze(1)
+                out[lo + t] = torch.einsum("hvk,hk->hv", S, q[t]).reshape(-1)
+            own.copy_(S)
+        return out.to(torch.float32 if A == torch.float32 else A)
+
     def argmax(self, logits):
         return logits.argmax(dim=-1).to(torch.int32)
 
