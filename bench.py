@@ -584,6 +584,72 @@ def sovezen_beside_others(args, dtype, item):
     return 0
 
 
+def nebutar_dict(width, ff, n_layers, heads, kv_heads, max_positions):
+    """A Nebutar of ``n_layers`` layers at a real model's layer sizes: attention (heads of 128) inside chunks of 1,024
+    positions beside the gated delta rule (width / 128 heads with a state of 128 x 128 over half as many key heads,
+    four taps), four copies of the stream, 32 silu-gated experts of a quarter of the dense size and 4 identity experts,
+    four per token."""
+    layer = {"type": "parallel",
+             "mixer": {"left": {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 50.0,
+                                "mask": {"size": 1024}},
+                       "right": {"heads": width // 128, "kv_heads": width // 256, "dim": 128, "vdim": 128, "conv": 4},
+                       "left_scale": 0.7, "right_scale": 0.7},
+             "mlp": {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 32, "identity": 4, "top": 4}}}
+    return {"architecture": "Nebutar", "vocab": 151936, "width": width, "layers": [json.loads(json.dumps(layer)) for _ in range(n_layers)],
+            "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0}, "max_positions": max_positions, "streams": 4}
+
+
+def nebutar_beside_others(args, dtype, item):
+    """Prefill and decode of Nebutar at a few real layer sizes, beside Pozalorn (the other model with two mixers side by
+    side and a recurrence), Tedulorn (routed experts) and Qwen3 of the same width, feed-forward size, vocabulary and
+    number of layers, all with the library's default solutions for its products. One JSON line of its own; the default
+    workload and its line are untouched."""
+    import torch
+    sizes = [("4b", "qwen3-4b"), ("8b", "qwen3-8b")]
+    n_layers = args.layers or 12
+    out = {"metric": "prefill and decode of Nebutar beside Pozalorn, Tedulorn and Qwen3 at equal width, feed-forward, vocabulary and layers",
+           "dtype": args.dtype, "layers": n_layers, "batch": args.batch, "context": args.context,
+           "prefill_tokens": args.prefill_tokens, "data": "synthetic: seeded random weights, uniform random token ids",
+           "sizes": {}}
+    only = set(filter(None, (args.only or "").split(",")))
+    names = ("nebutar", "pozalorn", "tedulorn", "qwen3")
+    for tag, preset in sizes:
+        if only & {name for name, _ in sizes} and tag not in only:
+            continue
+        q = preset_dict(preset)
+        q["num_hidden_layers"] = n_layers
+        shape = (q["hidden_size"], q["intermediate_size"], n_layers, q["num_attention_heads"], q["num_key_value_heads"])
+        cfgs = {"nebutar": nebutar_dict(*shape, args.max_len), "pozalorn": pozalorn_dict(*shape), "tedulorn": tedulorn_dict(*shape),
+                "qwen3": q}
+        point = {}
+        for name in names:
+            if only & set(names) and name not in only:
+                continue
+            cfg = cfgs[name]
+            config, engine = build_engine(cfg, dtype, args.batch, args.max_len, seed=0, compile_=not args.no_graphs,
+                                          chunk=max(2048, args.prefill_tokens), block_size=args.block_size)
+            for item_ in args.set:
+                key, _, value = item_.partition("=")
+                setattr(engine.runner.ops, key, json.loads(value))
+            V = cfg.get("vocab_size") or cfg["vocab"]
+            tok_s, ms = decode_rate(engine, args.batch, args.context, args.steps, args.warmup, V, seed=1)
+            pre_s = prefill_rate(engine, args.prefill_tokens, V, seed=2)
+            weights = (config.step_weight_bytes(args.batch, item) if hasattr(config, "step_weight_bytes")
+                       else config.param_counts()["read_per_step"] * item)
+            cache = (args.batch * args.context * config.kv_bytes_per_token(item) if name == "qwen3"
+                     else config.step_cache_bytes(args.batch, args.context, item))
+            point[name] = {"decode_tok_s": round(tok_s, 1), "decode_ms": round(ms, 4),
+                           "decode_hbm_frac": round((weights + cache) / (ms * 1e-3) / 1e9 / HBM_GBPS, 4),
+                           "prefill_ms": round(pre_s * 1e3, 3), "prefill_tok_s": round(args.prefill_tokens / pre_s, 1),
+                           "prefill_flop_frac": round(config.prefill_flops(args.prefill_tokens) / pre_s / PEAK_FLOPS[args.dtype], 4),
+                           "weights_gb": round(weights / 1e9, 3)}
+            release(engine)
+            torch.cuda.synchronize()
+        out["sizes"][tag] = point
+    print(json.dumps(out))
+    return 0
+
+
 def main(argv=None):
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -615,9 +681,12 @@ def main(argv=None):
     ap.add_argument("--sovezen", action="store_true",
                     help="instead of the default workload: prefill and decode of Sovezen at 4B- and 8B-sized layers "
                          "(--layers of them, default 12), each beside Mitisun, Tedulorn and Qwen3 of the same sizes")
+    ap.add_argument("--nebutar", action="store_true",
+                    help="instead of the default workload: prefill and decode of Nebutar at 4B- and 8B-sized layers "
+                         "(--layers of them, default 12), each beside Pozalorn, Tedulorn and Qwen3 of the same sizes")
     ap.add_argument("--only", default=None,
-                    help="--tedulorn, --pozalorn, --berelorn, --sovezen: sizes and models to run, with commas "
-                         "(4b,8b,sovezen,berelorn,pozalorn,tedulorn,mitisun,qwen3)")
+                    help="--tedulorn, --pozalorn, --berelorn, --sovezen, --nebutar: sizes and models to run, with commas "
+                         "(4b,8b,nebutar,sovezen,berelorn,pozalorn,tedulorn,mitisun,qwen3)")
     ap.add_argument("--dtype", choices=["bf16", "fp32"], default="bf16")
     ap.add_argument("--block-size", type=int, default=16, help="tokens per page of the cache (the reference's 16)")
     ap.add_argument("--no-graphs", action="store_true")
@@ -655,6 +724,8 @@ def main(argv=None):
         return berelorn_beside_others(args, dtype, item)
     if args.sovezen:
         return sovezen_beside_others(args, dtype, item)
+    if args.nebutar:
+        return nebutar_beside_others(args, dtype, item)
     if args.mixed:
         args.preset = args.preset or MIXED_PRESET
         args.max_len = max(args.max_len, 8192)

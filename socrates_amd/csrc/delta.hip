@@ -14,11 +14,12 @@ __device__ __forceinline__ float dl_sigmoid(float x) { return 1.f / (1.f + expf(
 // the step's last taps - 1 inputs) and silu. q and k become unit vectors per head, q also times q_scale: qk float32
 // [N, 2, G, Dp], zeros behind D. v in the compute dtype [N, H Dv]. z float32 [N, 2 H] holds the logits of beta and,
 // behind them, of the decay: gates float32 [N, H, 2] = (g, beta), g = exp(-exp(a_log) softplus(z + dt_bias)).
-// Grid (2 G + H + 1 roles, chunks of DL_CHUNK tokens, sequences); a wave takes a token of its role's vector at a time.
-// Only a sequence's first chunk reads and writes the state (taps - 1 <= DL_CHUNK).
-constexpr int DL_CHUNK = 32;
+// Grid (2 G + H + 1 roles, chunks of DL_CHUNK tokens, sequences). A wave takes DL_RUN tokens in a row of its role's vector:
+// with TAPS > 0 (the number of taps, up to 4) it loads all their inputs at once, each once; TAPS 0: any number of taps,
+// token by token. Only a sequence's first chunk reads and writes the state (taps - 1 <= DL_CHUNK).
+constexpr int DL_CHUNK = 32, DL_RUN = 8;
 
-template <typename T>
+template <typename T, int TAPS, int NJ>
 __global__ void __launch_bounds__(256)
 delta_prepare_kernel(const T* __restrict__ x, int ldx, int col, int G, int H, int D, int Dv, int Dp, const float* __restrict__ taps_w,
                      int taps, float q_scale, float unit_eps, const float* __restrict__ z, const float* __restrict__ a_log,
@@ -43,7 +44,8 @@ delta_prepare_kernel(const T* __restrict__ x, int ldx, int col, int G, int H, in
     const bool is_v = role >= 2 * G;
     const int dim = is_v ? Dv : D, C = 2 * G * D + H * Dv;
     const int c0 = is_v ? 2 * G * D + (role - 2 * G) * Dv : role * D;      // first channel of the role's vector
-    const int lane = threadIdx.x % SOC_WAVE, wave = threadIdx.x / SOC_WAVE, waves = blockDim.x / SOC_WAVE, back = taps - 1;
+    const int lane = threadIdx.x % SOC_WAVE, waves = blockDim.x / SOC_WAVE, back = taps - 1;
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / SOC_WAVE);
     float* kept = state + (size_t)seq_rows[seq] * stride + offset;
     auto channel = [&](int n, int c) {
         float y = 0.f;
@@ -54,6 +56,67 @@ delta_prepare_kernel(const T* __restrict__ x, int ldx, int col, int G, int H, in
         }
         return y * dl_sigmoid(y);
     };
+    if constexpr (TAPS > 0) {
+        // pieces of 64 NJ channels (a q or k vector is one piece: its norm is taken of the wave's registers)
+        const int n0 = first + wave * DL_RUN, n1 = min(n0 + DL_RUN, last);
+        for (int i0 = 0; n0 < n1 && i0 < dim; i0 += 64 * NJ) {
+            float in[DL_RUN + TAPS - 1][NJ], w[NJ][TAPS];
+            // (every load stands on its own, with what lies outside the step redirected to a row of it: no branches)
+#pragma unroll
+            for (int r = 0; r < DL_RUN + TAPS - 1; ++r) {
+                const T* row = x + (size_t)min(max(n0 - back + r, lo), n1 - 1) * ldx + col + c0;
+#pragma unroll
+                for (int j = 0; j < NJ; ++j) in[r][j] = to_float(row[min(i0 + lane + 64 * j, dim - 1)]);
+            }
+            if (n0 - lo < back) {                               // the sequence's first tokens: inputs of earlier steps
+#pragma unroll
+                for (int r = 0; r < TAPS - 1; ++r) {
+                    const int idx = n0 - lo - back + r;
+                    if (idx < 0) {
+#pragma unroll
+                        for (int j = 0; j < NJ; ++j) in[r][j] = kept[(size_t)(back + idx) * C + c0 + min(i0 + lane + 64 * j, dim - 1)];
+                    }
+                }
+            }
+#pragma unroll
+            for (int j = 0; j < NJ; ++j) {
+#pragma unroll
+                for (int k = 0; k < TAPS; ++k) {
+                    const int i = i0 + lane + 64 * j;
+                    const float t = taps_w[(size_t)(c0 + min(i, dim - 1)) * TAPS + k];
+                    w[j][k] = i < dim ? t : 0.f;                // (channels beyond the vector come out as zeros)
+                }
+            }
+#pragma unroll
+            for (int r = 0; r < DL_RUN; ++r) {
+                if (n0 + r < n1) {
+                    float y[NJ], ss = 0.f;
+#pragma unroll
+                    for (int j = 0; j < NJ; ++j) {
+                        float a = 0.f;
+#pragma unroll
+                        for (int k = 0; k < TAPS; ++k) a = fmaf(w[j][k], in[r + k][j], a);
+                        y[j] = a * dl_sigmoid(a);
+                        ss = fmaf(y[j], y[j], ss);
+                    }
+                    const size_t n = n0 + r;
+                    if (is_v) {
+#pragma unroll
+                        for (int j = 0; j < NJ; ++j) {
+                            const int i = i0 + lane + 64 * j;
+                            if (i < dim) v_out[n * H * Dv + (size_t)(role - 2 * G) * Dv + i] = from_float<T>(y[j]);
+                        }
+                    } else {
+                        const float inv = 1.f / sqrtf(wave_sum(ss) + unit_eps) * (role < G ? q_scale : 1.f);
+                        float* dst = qk + (n * 2 * G + role) * Dp;
+#pragma unroll
+                        for (int j = 0; j < NJ; ++j)
+                            if (lane + 64 * j < Dp) dst[lane + 64 * j] = y[j] * inv;
+                    }
+                }
+            }
+        }
+    } else
     for (int n = first + wave; n < last; n += waves) {
         if (is_v) {
             for (int i = lane; i < dim; i += SOC_WAVE) v_out[(size_t)n * H * Dv + (role - 2 * G) * Dv + i] = from_float<T>(channel(n, c0 + i));
@@ -94,12 +157,17 @@ SOC_EXPORT int soc_delta_prepare(const void* x, int ldx, int col, int G, int H, 
         max_q_len < 1)
         return (int)hipErrorInvalidValue;
     const dim3 grid(2 * G + H + 1, (max_q_len + DL_CHUNK - 1) / DL_CHUNK, n_seqs), block(max_q_len == 1 ? 64 : 256);
-    if (dtype == 0)
-        hipLaunchKernelGGL(delta_prepare_kernel<float>, grid, block, 0, stream, (const float*)x, ldx, col, G, H, D, Dv, Dp, taps_w, taps,
-                           q_scale, unit_eps, z, a_log, dt_bias, state, (size_t)stride, offset, seq_qstart, seq_rows, qk, (float*)v_out, gates);
-    else
-        hipLaunchKernelGGL(delta_prepare_kernel<bf16>, grid, block, 0, stream, (const bf16*)x, ldx, col, G, H, D, Dv, Dp, taps_w, taps,
-                           q_scale, unit_eps, z, a_log, dt_bias, state, (size_t)stride, offset, seq_qstart, seq_rows, qk, (bf16*)v_out, gates);
+#define SOC_DP(T, TAPS, NJ)                                                                                                      \
+    hipLaunchKernelGGL((delta_prepare_kernel<T, TAPS, NJ>), grid, block, 0, stream, (const T*)x, ldx, col, G, H, D, Dv, Dp, taps_w, taps, \
+                       q_scale, unit_eps, z, a_log, dt_bias, state, (size_t)stride, offset, seq_qstart, seq_rows, qk, (T*)v_out, gates)
+#define SOC_DP_T(T)                                                                                                     \
+    if (taps == 4) { if (D <= 64) SOC_DP(T, 4, 1); else if (D <= 128) SOC_DP(T, 4, 2); else SOC_DP(T, 4, 4); }          \
+    else if (taps == 3) { if (D <= 128) SOC_DP(T, 3, 2); else SOC_DP(T, 3, 4); }                                        \
+    else if (taps == 2) { if (D <= 128) SOC_DP(T, 2, 2); else SOC_DP(T, 2, 4); }                                        \
+    else SOC_DP(T, 0, 4);
+    if (dtype == 0) { SOC_DP_T(float) } else { SOC_DP_T(bf16) }
+#undef SOC_DP_T
+#undef SOC_DP
     return soc_last_error();
 }
 

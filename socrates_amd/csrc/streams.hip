@@ -69,14 +69,28 @@ __device__ __forceinline__ void stream_in(const StreamIn& b, int n, size_t total
     if (b.top > 0) {
 #pragma unroll
         for (int e = 0; e < V; ++e) x[e] = 0.f;
-        for (int r = 0; r < b.top; ++r) {
-            float t[V];
-            const float w = b.weight[(size_t)n * b.top + r];
-            const int at = b.place[(size_t)n * b.top + r];
-            if (at >= 0) VecLoad<float, V>::load((const float*)b.y + (size_t)at * d + c, t);
-            else VecLoad<T, V>::load((const T*)b.through + (size_t)n * d + c, t);
+        float same[V];                                          // (read once, so that the loads below need no branch)
 #pragma unroll
-            for (int e = 0; e < V; ++e) x[e] = fmaf(w, t[e], x[e]);
+        for (int e = 0; e < V; ++e) same[e] = 0.f;
+        if (b.through) VecLoad<T, V>::load((const T*)b.through + (size_t)n * d + c, same);
+        for (int r0 = 0; r0 < b.top; r0 += 4) {                 // four at a time: their loads are on the way together
+            float t[4][V], w[4];
+            int at[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const size_t i = (size_t)n * b.top + min(r0 + r, b.top - 1);
+                at[r] = b.place[i];
+                w[r] = b.weight[i];
+            }
+#pragma unroll
+            for (int r = 0; r < 4; ++r) VecLoad<float, V>::load((const float*)b.y + (size_t)max(at[r], 0) * d + c, t[r]);
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                if (r0 + r < b.top) {
+#pragma unroll
+                    for (int e = 0; e < V; ++e) x[e] = fmaf(w[r], at[r] >= 0 ? t[r][e] : same[e], x[e]);
+                }
+            }
         }
     } else if (b.parts > 0) {
         VecLoad<float, V>::load((const float*)b.y + (size_t)n * d + c, x);
@@ -105,10 +119,10 @@ struct StreamNorm {
 // One workgroup per row of out. x float32 [N, S, d]. With a.y: the old copies x_s and y = a (+ b) give
 // x_t <- sum_s mix[s, t] x_s + out_w[t] y (mix null: x_t <- x_t + y). Then u = sum_t read[t] x_t (read null: plain
 // sum), normed into out (no gain: nothing more). Without a.y nothing is written to x, and rows (null: all) selects the
-// rows of x that are read. PER pieces of V elements per thread, the combination staying in registers; PER 0: any number of
+// rows of x that are read. NT threads, PER pieces of V elements per thread, the combination staying in registers; PER 0: any number of
 // pieces, the combination in LDS (d floats, every thread its own).
-template <typename T, int SP, int V, int PER>
-__global__ void __launch_bounds__(256)
+template <typename T, int SP, int V, int PER, int NT>
+__global__ void __launch_bounds__(NT)
 streams_kernel(float* __restrict__ x, int S, StreamIn a, StreamIn b, const float* __restrict__ mix, const float* __restrict__ out_w,
                const float* __restrict__ read, StreamNorm norm, const int* __restrict__ rows, T* __restrict__ out, int N, int d) {
     __shared__ float scratch[16];
@@ -167,11 +181,11 @@ streams_kernel(float* __restrict__ x, int S, StreamIn a, StreamIn b, const float
         if constexpr (PER > 0) {
 #pragma unroll
             for (int i = 0; i < PER; ++i) {
-                const int c = (threadIdx.x + i * 256) * V;
+                const int c = (threadIdx.x + i * NT) * V;
                 if (c < d) f(c, kept[i]);
             }
         } else {
-            for (int c = threadIdx.x * V; c < d; c += 256 * V) {
+            for (int c = threadIdx.x * V; c < d; c += NT * V) {
                 float u[V];
 #pragma unroll
                 for (int e = 0; e < V; ++e) u[e] = held[c + e];
@@ -207,19 +221,22 @@ streams_kernel(float* __restrict__ x, int S, StreamIn a, StreamIn b, const float
 template <typename T, int SP>
 static int launch_streams(float* x, int S, const StreamIn& a, const StreamIn& b, const float* mix, const float* out_w, const float* read,
                           const StreamNorm& norm, const int* rows, void* out, int N, int n_out, int d, hipStream_t stream) {
-#define SOC_ST(SPV, V, PER)                                                                                                      \
-    hipLaunchKernelGGL((streams_kernel<T, SPV, V, PER>), dim3(n_out), dim3(256), (PER) ? 0 : d * sizeof(float), stream, x, S, a, b, mix, \
+#define SOC_ST(SPV, V, PER, NT)                                                                                                      \
+    hipLaunchKernelGGL((streams_kernel<T, SPV, V, PER, NT>), dim3(n_out), dim3(NT), (PER) ? 0 : d * sizeof(float), stream, x, S, a, b, mix, \
                        out_w, read, norm, rows, (T*)out, N, d)
     if (d > 16000) return (int)hipErrorInvalidValue;            // (what LDS holds)
     if constexpr (SP <= 4) {
-        if (d % 4 == 0 && d <= 1024) { SOC_ST(SP, 4, 1); return soc_last_error(); }
-        if (d % 4 == 0 && d <= 2048) { SOC_ST(SP, 4, 2); return soc_last_error(); }
-        if (d % 4 == 0 && d <= 3072) { SOC_ST(SP, 4, 3); return soc_last_error(); }
-        if (d % 4 == 0 && d <= 4096) { SOC_ST(SP, 4, 4); return soc_last_error(); }
+        if (d % 4 == 0 && d <= 1024) { SOC_ST(SP, 4, 1, 256); return soc_last_error(); }
+        // (few rows: a row's pieces side by side, not one behind the other)
+        if (d % 4 == 0 && d <= 2048 && n_out <= 512) { SOC_ST(SP, 4, 1, 512); return soc_last_error(); }
+        if (d % 4 == 0 && d <= 4096 && n_out <= 512) { SOC_ST(SP, 4, 1, 1024); return soc_last_error(); }
+        if (d % 4 == 0 && d <= 2048) { SOC_ST(SP, 4, 2, 256); return soc_last_error(); }
+        if (d % 4 == 0 && d <= 3072) { SOC_ST(SP, 4, 3, 256); return soc_last_error(); }
+        if (d % 4 == 0 && d <= 4096) { SOC_ST(SP, 4, 4, 256); return soc_last_error(); }
     }
     constexpr int SPG = SP <= 4 ? 4 : 16;
-    if (d % 4 == 0) SOC_ST(SPG, 4, 0);
-    else SOC_ST(SPG, 1, 0);
+    if (d % 4 == 0) SOC_ST(SPG, 4, 0, 256);
+    else SOC_ST(SPG, 1, 0, 256);
 #undef SOC_ST
     return soc_last_error();
 }

@@ -24,6 +24,7 @@ def _state_layout(spec: GatedDeltaSpec):
 
 class GatedDelta:
     takes_out_dtype = True      # forward(..., out_dtype=): the dtype of its last product
+    takes_partial = True
     takes_first = True          # forward(..., first=): (rows, column) of ``w_first``'s product, taken by the caller
 
     @staticmethod
@@ -51,7 +52,8 @@ class GatedDelta:
         self.w_o = tensors["o"]
         self.state_at = _state_layout(spec)[0]
 
-    def forward(self, x, ctx, slot, write=True, out_dtype=None, first=None):
+    def forward(self, x, ctx, slot, write=True, out_dtype=None, first=None, partial=False):
+        """``first``: see ``takes_first``; ``partial``: the result may come as float32 partial sums [S, N, hidden]."""
         s, ops = self.spec, self.ops
         H, inner = s.n_heads, s.n_heads * s.v_dim
         if not write:
@@ -61,7 +63,7 @@ class GatedDelta:
         raw = ops.delta_rule(first, at + inner, s.n_kv_heads, H, s.head_dim, s.v_dim, self.taps, float(s.head_dim) ** -0.5,
                              s.unit_eps, z, self.a_log, self.dt_bias, slot.state, 0, self.state_at, ctx)
         o = ops.gated_group_norm(raw, first[:, at:at + inner], self.gain, H, s.eps, gate_first=False)
-        return ops.linear(o, self.w_o, out_dtype=out_dtype)
+        return ops.linear(o, self.w_o, out_dtype=out_dtype, **({"allow_partial": True} if partial else {}))
 
 
 register_part(GatedDeltaSpec, GatedDelta)

@@ -55,7 +55,7 @@ class ParallelMixer:
     def forward(self, x, ctx, slot, write=True, apart=False):
         """``apart``: return [(left, its scale), (right, its scale)] where no bias is left to add."""
         s, ops = self.spec, self.ops
-        left, right = {}, {}
+        left, right = ({"partial": True} if apart and getattr(p, "takes_partial", False) else {} for p in (self.left, self.right))
         if self.w_first is not None:
             first = ops.linear(x, self.w_first)
             left["first"], right["first"] = (first, 0), (first, self.cut)

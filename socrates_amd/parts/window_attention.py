@@ -30,6 +30,7 @@ def pair_frequencies(position, device):
 
 class WindowAttention:
     takes_out_dtype = True      # forward(..., out_dtype=): the dtype of its last product
+    takes_partial = True        # forward(..., partial=True): its last product may come as partial sums
     offers_raw = True           # forward(..., raw=True): (last product, its bias) with the bias left to the caller
 
     @staticmethod
@@ -91,9 +92,9 @@ class WindowAttention:
         # a caller may take the first product with other rows (the bias then does not fit its columns)
         self.takes_first = self.bias is None
 
-    def forward(self, x, ctx, slot, write=True, out_dtype=None, raw=False, first=None):
+    def forward(self, x, ctx, slot, write=True, out_dtype=None, raw=False, first=None, partial=False):
         """``raw``: return (product, the output projection's bias or None) and leave the bias to the caller. ``first`` =
-        (rows, column): ``w_first``'s product is in these rows from that column on, the caller has taken it."""
+        (rows, column): ``w_first``'s product is in these rows from that column on, the caller has taken it. ``partial``: the result may come as float32 partial sums [S, N, hidden]."""
         s, ops = self.spec, self.ops
         H, G, D, Dv, P = s.n_heads, s.n_kv_heads, s.head_dim, s.v_dim, s.cache_width
         if not write:
@@ -120,7 +121,7 @@ class WindowAttention:
             o = ops.head_gate(o, H, P, Dv, first[:, at + self.col_gate:at + self.col_gate + H])
         elif self.value_freq is not None or P != Dv:
             o = ops.turn_back(o, H, P, Dv, self.value_freq, ctx.positions)
-        y = ops.linear(o, self.w_o, out_dtype=out_dtype)
+        y = ops.linear(o, self.w_o, out_dtype=out_dtype, **({"allow_partial": True} if partial and self.o_bias is None else {}))
         if raw:
             return y, self.o_bias
         return y if self.o_bias is None else ops.scaled_sum(y, 1.0, None, 0.0, self.o_bias)
