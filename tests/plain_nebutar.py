@@ -64,12 +64,10 @@ def delta_walk(q, k, v, g, beta, state=None):
     S = torch.zeros(H, D, v.shape[-1], dtype=q.dtype) if state is None else state.clone()
     out = torch.empty_like(v)
     for t in range(T):
-        for h in range(H):
-            s = g[t, h] * S[h]
-            u = beta[t, h] * (v[t, h] - s.T @ k[t, h])
-            s = s + torch.outer(k[t, h], u)
-            out[t, h] = s.T @ q[t, h]
-            S[h] = s
+        S = g[t].view(H, 1, 1) * S
+        u = beta[t].view(H, 1) * (v[t] - (S * k[t].unsqueeze(-1)).sum(1))          # S^T k, head by head
+        S = S + k[t].unsqueeze(-1) * u.unsqueeze(1)
+        out[t] = (S * q[t].unsqueeze(-1)).sum(1)
     return out, S
 
 
