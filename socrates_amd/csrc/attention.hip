@@ -702,6 +702,7 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_po
 #pragma unroll
             for (int kk = 0; kk < QK_STEPS; ++kk)
                 s = qk_mfma(k_ok ? kf.v[kk] : make_uint4(0u, 0u, 0u, 0u), qf[rt][kk], s);
+            const int last_seen = min(row_pos[rt], hi - 1), first_key_seen = max(row_first[rt], lo_seen);
             float sv[4];
             float mx = -INFINITY;                           // of the raw scores: the scale is positive
             if constexpr (CAP) {                            // (a form of its own: a layer without a cap pays nothing)
@@ -712,9 +713,10 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_po
             for (int r = 0; r < 4; ++r) {
                 sv[r] = s[r];
                 if constexpr (MASKED) {
+                    // (no branch here: between a product and what reads its result the compiler counts the wait
+                    // states along one way round a branch only, and on the other the result is read too early)
                     const int key = key0 + 4 * kb + r;
-                    bool seen = key <= row_pos[rt] && key < hi && key >= lo_seen;
-                    if (window != 0) seen = seen && key >= row_first[rt];
+                    const bool seen = (key <= last_seen) & (key >= first_key_seen);
                     sv[r] = seen ? sv[r] : -INFINITY;
                 }
                 mx = fmaxf(mx, sv[r]);
@@ -1377,6 +1379,9 @@ paged_attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k
                 s0 = qk_mfma(ka[kk], qf[rt][kk], s0);
                 s1 = qk_mfma(kc[kk], qf[rt][kk], s1);
             }
+            // (of means: every entry up to the row's last)
+            const int last_seen = key0 < 0 ? mean_end[rt] - 1 : row_pos[rt];
+            const int first_seen_key = key0 < 0 ? key0 : row_first[rt], kept_seen = key0 < 0 ? key0 : keep_first;
             float t[8];
             float mx = -INFINITY;                           // of the raw scores: the scale is positive
             if constexpr (CAP) {                            // (a form of its own: a layer without a cap pays nothing)
@@ -1387,10 +1392,10 @@ paged_attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k
             for (int r = 0; r < 8; ++r) {
                 t[r] = r < 4 ? s0[r & 3] : s1[r & 3];
                 if constexpr (MASKED) {
+                    // (no branch, see the per-wave kernel; a tile of means, uniform, has negative keys, and without a
+                    // window row_first is 0)
                     const int key = key0 + 8 * kb + r;
-                    bool seen = key <= row_pos[rt];
-                    if (window != 0) seen = seen && (key >= row_first[rt] || key < keep_first);
-                    if (key0 < 0) seen = key < mean_end[rt];          // (uniform: a tile of means)
+                    const bool seen = (key <= last_seen) & ((key >= first_seen_key) | (key < kept_seen));
                     t[r] = seen ? t[r] : -INFINITY;
                 }
                 mx = fmaxf(mx, t[r]);
@@ -1450,6 +1455,8 @@ paged_attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k
             sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8_t*>(&ka),
                                                          *reinterpret_cast<const bf16x8_t*>(&qf32[t]), sc, 0, 0, 0);
         }
+        const int last_seen = key0 < 0 ? mean_end32 - 1 : row_pos32;
+        const int first_seen_key = key0 < 0 ? key0 : row_first32, kept_seen = key0 < 0 ? key0 : keep_first;
         float mx = -INFINITY;                               // of the raw scores: the scale is positive
         if constexpr (CAP) {                                // (a form of its own: a layer without a cap pays nothing)
 #pragma unroll
@@ -1458,10 +1465,8 @@ paged_attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
             if constexpr (MASKED) {
-                const int key = key0 + 16 * (i / 8) + 8 * g32 + i % 8;
-                bool seen = key <= row_pos32;
-                if (window != 0) seen = seen && (key >= row_first32 || key < keep_first);
-                if (key0 < 0) seen = key < mean_end32;               // (uniform: a tile of means)
+                const int key = key0 + 16 * (i / 8) + 8 * g32 + i % 8;       // (no branch, see the per-wave kernel)
+                const bool seen = (key <= last_seen) & ((key >= first_seen_key) | (key < kept_seen));
                 sc[i] = seen ? sc[i] : -INFINITY;
             }
             mx = fmaxf(mx, sc[i]);

@@ -145,10 +145,19 @@ def random_weights(cfg, seed):
     return out
 
 
-def write_model(folder, cfg, seed, weights=None):
+def settled(w, seed):
+    """The same weights with corrections so far apart that no choice of experts hangs on a rounding (scores lie between 0
+    and 1): what bfloat16 does to a model whose recurrences would carry one other choice on to every later token."""
+    g = torch.Generator().manual_seed(seed)
+    return {k: 1.5 * torch.randperm(len(v), generator=g).float() - 2.0 if k.endswith(".correction") else v for k, v in w.items()}
+
+
+def write_model(folder, cfg, seed, weights=None, settle=False):
     folder = Path(folder)
     folder.mkdir(parents=True, exist_ok=True)
     weights = weights if weights is not None else random_weights(cfg, seed)
+    if settle:
+        weights = settled(weights, seed)
     (folder / "config.json").write_text(json.dumps(cfg))
     save_file({k: v.to(torch.bfloat16).contiguous() for k, v in weights.items()}, str(folder / "model.safetensors"))
     return folder
