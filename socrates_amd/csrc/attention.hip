@@ -3,7 +3,7 @@
 //
 // paged_attn_token_kernel: one workgroup per (token, kv head, query-head chunk, key
 // split). A query token at position p of cache row r attends to the keys lo..p of that
-// row (lo = 0, or p - window + 1 with a window), read through the row's block table.
+// row (lo = 0, p - window + 1 with a window, or the start of p's chunk), read through the row's block table.
 // It serves single decoded tokens and tokens of prompt portions alike, in float32 and
 // bfloat16. The reference's decode kernel (model/kernels/csrc/paged_attention.cu:65-274)
 // has the same task for one token per row; this one is laid out for 64-wide waves:

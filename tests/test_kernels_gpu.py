@@ -617,8 +617,8 @@ def test_attention_walks_of_large_heads_over_pages_of_any_size(kernel_sets, D, b
     """Head sizes above 128 with pages that hold no multiple of 16 keys (every lane looks its own
     key's page up), walks long enough for the loop over rounds of three tiles, with one split and
     with several, a decoded token and a portion; a large scale, so that a key read from the
-    wrong place shows (a reordering of this kernel's first loads once gave wrong sums in just
-    this corner, and nothing in the tests came near it)."""
+    wrong place shows (twice a change elsewhere in this kernel gave wrong sums in just this
+    corner: a branch behind the score product let its result be read too early)."""
     hip, _ = kernel_sets[torch.bfloat16]
     lens = [1116, 100, 203]
     slot, dense = make_paged_case(lens, 8, 2, D, bs, torch.bfloat16, seed=D + bs)
